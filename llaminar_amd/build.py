@@ -7,10 +7,15 @@ for gfx950 without a GPU, so this runs anywhere the ROCm toolchain is present.
 The host-side operator (``csrc/host``) is linked into a second library,
 ``libllaminar_ql_host.so``, on top of the first.
 
-Usage: ``python -m llaminar_amd.build``
+Sequence models (``csrc/seq``: kernels, operators and step driver over plain bf16 weights)
+are a library of their own, ``libllaminar_seq.so``, which needs neither of the others: with
+the sampler and the error plumbing it shares with them it builds in well under a minute.
+
+Usage: ``python -m llaminar_amd.build [--incremental] [--seq-only]``
 """
 from __future__ import annotations
 
+import fcntl
 import os
 import re
 import shutil
@@ -25,6 +30,7 @@ CSRC = PKG / "csrc"
 LIBDIR = PKG / "lib"
 LIB = LIBDIR / "libllaminar_ql.so"
 HOST_LIB = LIBDIR / "libllaminar_ql_host.so"
+SEQ_LIB = LIBDIR / "libllaminar_seq.so"
 OBJDIR = PKG / "build"
 
 ARCH = "gfx950"
@@ -187,6 +193,11 @@ def sources() -> list[Path]:
     return sorted(list(CSRC.glob("*.hip")) + list(CSRC.glob("*.cpp")))
 
 
+def seq_sources() -> list[Path]:
+    seq = CSRC / "seq"
+    return sorted(list(seq.glob("*.hip")) + list(seq.glob("*.cpp"))) + [CSRC / "ql_common.hip", CSRC / "sampling.hip"]
+
+
 def _deps_mtime() -> float:
     files = [f for f in CSRC.rglob("*") if f.is_file()] + list((ROOT / "include" / "llaminar_amd").glob("*.h*"))
     return max(f.stat().st_mtime for f in files)
@@ -223,7 +234,7 @@ def _drop_resource_remarks(lines: list[str]) -> list[str]:
 
 
 def _headers_mtime() -> float:
-    files = list(CSRC.glob("*.h")) + list((ROOT / "include" / "llaminar_amd").glob("*.h*"))
+    files = list(CSRC.glob("*.h")) + list((CSRC / "seq").glob("*.h")) + list((ROOT / "include" / "llaminar_amd").glob("*.h*"))
     return max(f.stat().st_mtime for f in files)
 
 
@@ -253,8 +264,40 @@ def _compile(src: Path, force: bool = True) -> Path:
     return obj
 
 
+def _link(objs: list[Path], lib: Path, verbose: bool) -> None:
+    # into a name of its own first: a process that loads the library meanwhile sees the old one or the new one
+    part = lib.with_suffix(f".{os.getpid()}.part")
+    cmd = [hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objs), f"-Wl,-soname,{lib.name}", "-o", str(part)]
+    proc = subprocess.run(cmd, capture_output=True, text=True)
+    if proc.returncode != 0:
+        part.unlink(missing_ok=True)
+        raise RuntimeError(f"link failed:\n{proc.stderr}")
+    part.replace(lib)
+    if verbose:
+        print(f"[llaminar_amd.build] wrote {lib} ({lib.stat().st_size} bytes)", flush=True)
+
+
+def build_seq(force: bool = True, verbose: bool = True) -> Path:
+    """Compile and link the sequence-model library alone.  With force=False an up-to-date one is kept."""
+    OBJDIR.mkdir(exist_ok=True)
+    LIBDIR.mkdir(exist_ok=True)
+    srcs = seq_sources()
+    with open(OBJDIR / ".seq.lock", "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)  # one builder at a time in a checkout
+        newest = max([f.stat().st_mtime for f in srcs] + [_headers_mtime()])
+        if not force and SEQ_LIB.exists() and SEQ_LIB.stat().st_mtime >= newest:
+            return SEQ_LIB
+        if verbose:
+            print(f"[llaminar_amd.build] hipcc {ARCH}: {len(srcs)} sources of the sequence models", flush=True)
+        with ThreadPoolExecutor(max_workers=min(8, len(srcs))) as pool:
+            objs = list(pool.map(lambda src: _compile(src, force), srcs))
+        _link(objs, SEQ_LIB, verbose)
+    return SEQ_LIB
+
+
 def build(force: bool = True, verbose: bool = True) -> Path:
-    """Compile and link the library.  With force=False an up-to-date library is kept."""
+    """Compile and link the libraries.  With force=False up-to-date ones are kept."""
+    build_seq(force, verbose)
     if not force and LIB.exists() and HOST_LIB.exists() and LIB.stat().st_mtime >= _deps_mtime():
         return LIB
     OBJDIR.mkdir(exist_ok=True)
@@ -264,15 +307,10 @@ def build(force: bool = True, verbose: bool = True) -> Path:
         print(f"[llaminar_amd.build] hipcc {ARCH}: {len(srcs)} sources", flush=True)
     with ThreadPoolExecutor(max_workers=min(8, len(srcs))) as pool:
         objs = list(pool.map(lambda src: _compile(src, force), srcs))
-    cmd = [hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objs), "-o", str(LIB)]
-    proc = subprocess.run(cmd, capture_output=True, text=True)
-    if proc.returncode != 0:
-        raise RuntimeError(f"link failed:\n{proc.stderr}")
-    if verbose:
-        print(f"[llaminar_amd.build] wrote {LIB} ({LIB.stat().st_size} bytes)", flush=True)
+    _link(objs, LIB, verbose)
     build_host(verbose)
     return LIB
 
 
 if __name__ == "__main__":
-    build(force="--incremental" not in sys.argv)
+    (build_seq if "--seq-only" in sys.argv else build)(force="--incremental" not in sys.argv)

@@ -1,0 +1,478 @@
+// Causal attention over a latent cache that serves as key and value at once, for gfx950.
+//
+// Queries arrive in latent space (q . W_uk, one vector of `rank` per head), so all heads of a
+// token share every cache row: a query row is a (token, head) pair, R = tokens * heads rows per
+// entry, all against the same keys.  A workgroup takes 16 WR rows and a stretch of the sequence,
+// walks it 32 WP positions at a time (WR * WP = 4 wavefronts), the cache rows staged once in LDS:
+//   scores  S[row][p] = sum_d q[row][d] c[p][d]   second operand: c rows as they lie
+//   output  O[row][d] = sum_p w[row][p] c[p][d]   second operand: c columns (transposing LDS read)
+// with a running maximum per row.  Softmax in 32-bit; for bf16 the weights enter the second
+// product as two bf16 pieces.  With WP > 1 the wavefronts of a row group split the positions and
+// merge through LDS; with several stretches per row group a second kernel merges those.
+#include "seq_common.h"
+#include "llaminar_amd/seq_api.h"
+
+namespace llamql
+{
+    constexpr int LAT_THREADS = 256;
+    constexpr int LAT_TARGET = 512; // workgroups aimed at before rows are no longer split
+
+    struct LatentArgs
+    {
+        const void *q;
+        const void *cache;
+        const int32_t *row0, *ntok, *slot, *pos;
+        int first, heads, rank, cap, chunk, nsplit, slices, rcap;
+        float scale;
+        void *o;
+        float *part_o, *part_ml;
+    };
+
+    // NOUT: 16-column output tiles of a wavefront.  QREG: the query rows stay in registers (rank <= 16 NOUT);
+    // otherwise they are read again for every stretch and blockIdx.z also counts output slices.
+    template <typename T, int NOUT, bool QREG, int WR>
+    __global__ void __launch_bounds__(LAT_THREADS)
+        latent_attention_kernel(LatentArgs p)
+    {
+        using O = Operand<T>;
+        using V = typename O::V;
+        constexpr int WP = 4 / WR, PT = 32 * WP;
+        constexpr int LPAD = 16 / sizeof(T);
+        constexpr int PW = sizeof(T) == 2 ? 2 : 1; // pieces of a softmax weight
+        constexpr int SLD = 36;
+        extern __shared__ __attribute__((aligned(16))) char smem[];
+        __shared__ __attribute__((aligned(16))) float s_p[4][16 * SLD];
+        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+        const int c = lane & 15, g = lane >> 4;
+        const int wr = wave % WR, wp = wave / WR;
+        const int ei = QREG ? blockIdx.z : blockIdx.z / p.slices;
+        const int slice = QREG ? 0 : blockIdx.z % p.slices;
+        const int e = p.first + ei, split = blockIdx.y;
+        const int R = p.ntok[e] * p.heads, pos0 = p.pos[e];
+        const int rb = blockIdx.x * 16 * WR;
+        if (rb >= R)
+            return;
+        const int last_row = rb + 16 * WR - 1 < R ? rb + 16 * WR - 1 : R - 1;
+        const int kmax = pos0 + last_row / p.heads; // newest position any row of the group sees
+        const int k0 = split * p.chunk;
+        if (k0 > kmax || kmax >= p.cap)
+            return;
+        const int k1 = k0 + p.chunk < kmax + 1 ? k0 + p.chunk : kmax + 1;
+
+        const int ksteps = p.rank >> 5;
+        const int ld = p.rank + LPAD;
+        T *tile = reinterpret_cast<T *>(smem);
+        const T *cache = static_cast<const T *>(p.cache) + (size_t)p.slot[e] * p.cap * p.rank;
+
+        const int qrow = rb + wr * 16 + c < R ? rb + wr * 16 + c : R - 1;
+        const T *q = static_cast<const T *>(p.q) + ((size_t)p.row0[e] * p.heads + qrow) * p.rank + 8 * g;
+        V qreg[QREG ? NOUT / 2 : 1];
+        if (QREG)
+        {
+#pragma unroll
+            for (int ks = 0; ks < NOUT / 2; ++ks)
+                if (ks < ksteps)
+                    qreg[ks] = O::load(q + ks * 32);
+        }
+        int limit[4]; // newest position of this lane's result rows 4 g + r
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+        {
+            const int row = rb + wr * 16 + 4 * g + r;
+            limit[r] = row < R ? pos0 + row / p.heads : -1;
+        }
+        const int out_tiles = (p.rank >> 4) - slice * NOUT < NOUT ? (p.rank >> 4) - slice * NOUT : NOUT;
+
+        float m[4], l[4];
+        f32x4 acc[NOUT];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+        {
+            m[r] = -INFINITY;
+            l[r] = 0.0f;
+        }
+#pragma unroll
+        for (int t = 0; t < NOUT; ++t)
+            acc[t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+
+        const int pieces = p.rank * (int)sizeof(T) / 16;
+        for (int kt = k0; kt < k1; kt += PT)
+        {
+            __syncthreads();
+            for (int r = threadIdx.x >> 3; r < PT; r += LAT_THREADS / 8)
+            {
+                const int pos = kt + r <= kmax ? kt + r : kmax; // rows past the end are masked; they only must be numbers
+                const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)pos * p.rank);
+                u32x4 *dst = reinterpret_cast<u32x4 *>(tile + r * ld);
+                for (int i = threadIdx.x & 7; i < pieces; i += 8)
+                    dst[i] = src[i];
+            }
+            __syncthreads();
+
+            const T *mine = tile + wp * 32 * ld;
+            f32x4 s[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
+            if (QREG)
+            {
+#pragma unroll
+                for (int ks = 0; ks < NOUT / 2; ++ks)
+                    if (ks < ksteps)
+                    {
+                        s[0] = O::mma(qreg[ks], O::load(mine + c * ld + ks * 32 + 8 * g), s[0]);
+                        s[1] = O::mma(qreg[ks], O::load(mine + (16 + c) * ld + ks * 32 + 8 * g), s[1]);
+                    }
+            }
+            else
+                for (int ks = 0; ks < ksteps; ++ks)
+                {
+                    const V a = O::load(q + ks * 32);
+                    s[0] = O::mma(a, O::load(mine + c * ld + ks * 32 + 8 * g), s[0]);
+                    s[1] = O::mma(a, O::load(mine + (16 + c) * ld + ks * 32 + 8 * g), s[1]);
+                }
+            float alpha[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+            {
+                const int pa = kt + wp * 32 + c;
+                const float sa = pa <= limit[r] ? s[0][r] * p.scale : -INFINITY;
+                const float sb = pa + 16 <= limit[r] ? s[1][r] * p.scale : -INFINITY;
+                float mx = fmaxf(sa, sb);
+#pragma unroll
+                for (int off = 1; off < 16; off <<= 1)
+                    mx = fmaxf(mx, __shfl_xor(mx, off, 64));
+                const float mn = fmaxf(m[r], mx);
+                const float base = mn == -INFINITY ? 0.0f : mn;
+                alpha[r] = expf(m[r] - base);
+                m[r] = mn;
+                const float ea = expf(sa - base), eb = expf(sb - base);
+                l[r] = l[r] * alpha[r] + ea + eb;
+                s_p[wave][(4 * g + r) * SLD + c] = ea;
+                s_p[wave][(4 * g + r) * SLD + 16 + c] = eb;
+            }
+            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+            __builtin_amdgcn_wave_barrier();
+            __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+            V w[PW];
+            {
+                const f32x4 a = *reinterpret_cast<const f32x4 *>(&s_p[wave][c * SLD + 8 * g]);
+                const f32x4 b = *reinterpret_cast<const f32x4 *>(&s_p[wave][c * SLD + 8 * g + 4]);
+                split_pieces<T, PW>(__builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7), w);
+            }
+#pragma unroll
+            for (int t = 0; t < NOUT; ++t)
+                if (t < out_tiles)
+                {
+                    const V v = load_columns(mine + (slice * NOUT + t) * 16, ld, lane);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        acc[t][r] *= alpha[r];
+#pragma unroll
+                    for (int i = 0; i < PW; ++i)
+                        acc[t] = O::mma(w[i], v, acc[t]);
+                }
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int off = 1; off < 16; off <<= 1)
+                l[r] += __shfl_xor(l[r], off, 64);
+
+        if (WP > 1)
+        {
+            // merge the wavefronts of each row group: [wave][16 rows][16 NOUT columns], then (m, l)
+            __syncthreads();
+            float *s_o = reinterpret_cast<float *>(smem);
+            float *s_ml = &s_p[0][0];
+            constexpr int OLD = NOUT * 16 + 4;
+#pragma unroll
+            for (int t = 0; t < NOUT; ++t)
+                if (t < out_tiles)
+                {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        s_o[(wave * 16 + 4 * g + r) * OLD + t * 16 + c] = acc[t][r];
+                }
+            if (c == 0)
+            {
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                {
+                    s_ml[(wave * 16 + 4 * g + r) * 2] = m[r];
+                    s_ml[(wave * 16 + 4 * g + r) * 2 + 1] = l[r];
+                }
+            }
+            __syncthreads();
+            for (int i = threadIdx.x; i < WR * 16 * out_tiles * 16; i += LAT_THREADS)
+            {
+                const int row = i / (out_tiles * 16), d = i - row * (out_tiles * 16); // row of the group
+                if (rb + row >= R)
+                    continue;
+                float M = -INFINITY;
+#pragma unroll
+                for (int w = 0; w < WP; ++w)
+                    M = fmaxf(M, s_ml[((w * WR * 16) + row) * 2]);
+                const float base = M == -INFINITY ? 0.0f : M;
+                float L = 0.0f, y = 0.0f;
+#pragma unroll
+                for (int w = 0; w < WP; ++w)
+                {
+                    const float f = expf(s_ml[((w * WR * 16) + row) * 2] - base);
+                    L += f * s_ml[((w * WR * 16) + row) * 2 + 1];
+                    y += f * s_o[(w * WR * 16 + row) * OLD + d];
+                }
+                const int col = slice * NOUT * 16 + d;
+                if (p.nsplit == 1)
+                    static_cast<T *>(p.o)[((size_t)p.row0[e] * p.heads + rb + row) * p.rank + col] = (T)(y / L);
+                else
+                {
+                    const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + rb + row;
+                    p.part_o[at * p.rank + col] = y;
+                    if (d == 0 && slice == 0)
+                    {
+                        p.part_ml[at * 2] = M;
+                        p.part_ml[at * 2 + 1] = L;
+                    }
+                }
+            }
+            return;
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+        {
+            const int row = rb + wr * 16 + 4 * g + r;
+            if (row >= R)
+                continue;
+            const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + row;
+            const float inv = 1.0f / l[r];
+#pragma unroll
+            for (int t = 0; t < NOUT; ++t)
+                if (t < out_tiles)
+                {
+                    const int col = (slice * NOUT + t) * 16 + c;
+                    if (p.nsplit == 1)
+                        static_cast<T *>(p.o)[((size_t)p.row0[e] * p.heads + row) * p.rank + col] = (T)(acc[t][r] * inv);
+                    else
+                        p.part_o[at * p.rank + col] = acc[t][r];
+                }
+            if (p.nsplit > 1 && c == 0 && slice == 0)
+            {
+                p.part_ml[at * 2] = m[r];
+                p.part_ml[at * 2 + 1] = l[r];
+            }
+        }
+    }
+
+    // one workgroup per query row: o = sum_s o_s e^(m_s - M) / sum_s l_s e^(m_s - M)
+    constexpr int LAT_MERGE_THREADS = 128;
+    template <typename T>
+    __global__ void __launch_bounds__(LAT_MERGE_THREADS)
+        latent_merge_kernel(LatentArgs p)
+    {
+        const int ei = blockIdx.y, e = p.first + ei, row = blockIdx.x;
+        if (row >= p.ntok[e] * p.heads)
+            return;
+        const int limit = p.pos[e] + row / p.heads;
+        if (limit >= p.cap)
+            return;
+        const int used = limit / p.chunk + 1;
+        const size_t at = (size_t)ei * p.nsplit * p.rcap + row;
+        float M = -INFINITY;
+        for (int s = 0; s < used; ++s)
+            M = fmaxf(M, p.part_ml[(at + (size_t)s * p.rcap) * 2]);
+        for (int d = threadIdx.x * 4; d < p.rank; d += LAT_MERGE_THREADS * 4)
+        {
+            float L = 0.0f;
+            f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll 4
+            for (int s = 0; s < used; ++s)
+            {
+                const size_t k = at + (size_t)s * p.rcap;
+                const float f = expf(p.part_ml[k * 2] - M);
+                L += f * p.part_ml[k * 2 + 1];
+                y = y + *reinterpret_cast<const f32x4 *>(p.part_o + k * p.rank + d) * f;
+            }
+            typedef T t4 __attribute__((ext_vector_type(4)));
+            *reinterpret_cast<t4 *>(static_cast<T *>(p.o) + ((size_t)p.row0[e] * p.heads + row) * p.rank + d) =
+                __builtin_convertvector(y * (1.0f / L), t4);
+        }
+    }
+
+    template <typename T>
+    __global__ void __launch_bounds__(256)
+        latent_append_kernel(const float *__restrict__ x, int ldx, const float *__restrict__ norm, float eps, int k_real,
+                             const int32_t *__restrict__ row_slot, const int32_t *__restrict__ row_pos,
+                             T *__restrict__ cache, int rank, int cap)
+    {
+        typedef T t4 __attribute__((ext_vector_type(4)));
+        __shared__ float s_sum[4];
+        const int m = blockIdx.x, pos = row_pos[m];
+        const f32x4 *row = reinterpret_cast<const f32x4 *>(x + (size_t)m * ldx);
+        float sum = 0.0f;
+        for (int i = threadIdx.x; i < rank / 4; i += 256)
+        {
+            const f32x4 v = row[i];
+            sum += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+        }
+        sum = block_sum<256>(sum, s_sum);
+        if (pos < 0 || pos >= cap)
+            return;
+        const float inv = 1.0f / sqrtf(sum / (float)k_real + eps);
+        T *dst = cache + ((size_t)row_slot[m] * cap + pos) * rank;
+        for (int i = threadIdx.x; i < rank / 4; i += 256)
+            *reinterpret_cast<t4 *>(dst + 4 * i) =
+                __builtin_convertvector(row[i] * inv * reinterpret_cast<const f32x4 *>(norm)[i], t4);
+    }
+
+    namespace
+    {
+        template <typename T, int NOUT, bool QREG, int WR>
+        bool latent_launch(const char *fn, const LatentArgs &p, int row_blocks, int n, hipStream_t st)
+        {
+            static LdsGrant grant;
+            constexpr int WP = 4 / WR;
+            size_t lds = (size_t)32 * WP * (p.rank + 16 / sizeof(T)) * sizeof(T);
+            const size_t merge = WP > 1 ? (size_t)64 * (NOUT * 16 + 4) * 4 : 0;
+            lds = lds > merge ? lds : merge;
+            constexpr size_t most = 150 * 1024;
+            if (lds > most)
+                return fail(fn, "rank=%d does not fit the LDS", p.rank);
+            if (lds > 48 * 1024 && allow_lds(grant, reinterpret_cast<const void *>(&latent_attention_kernel<T, NOUT, QREG, WR>), most) != hipSuccess)
+                return fail(fn, "cannot reserve %zu bytes of LDS", lds);
+            hipLaunchKernelGGL((latent_attention_kernel<T, NOUT, QREG, WR>), dim3(row_blocks, p.nsplit, n * p.slices),
+                               dim3(LAT_THREADS), lds, st, p);
+            return launched(fn);
+        }
+        template <typename T, int NOUT, bool QREG>
+        bool latent_rows(const char *fn, const LatentArgs &p, int wr, int row_blocks, int n, hipStream_t st)
+        {
+            if (wr == 1)
+                return latent_launch<T, NOUT, QREG, 1>(fn, p, row_blocks, n, st);
+            if (wr == 2)
+                return latent_launch<T, NOUT, QREG, 2>(fn, p, row_blocks, n, st);
+            return latent_launch<T, NOUT, QREG, 4>(fn, p, row_blocks, n, st);
+        }
+
+        // how a call is cut up: wavefronts per row group and stretches of the sequence
+        struct LatentPlan
+        {
+            int wr, row_blocks, chunk, nsplit;
+        };
+        LatentPlan latent_plan(int n, int max_ntok, int max_len, int heads, int rank, int elem)
+        {
+            LatentPlan pl{};
+            const int R = max_ntok * heads;
+            pl.wr = R <= 16 ? 1 : R <= 32 ? 2 : 4;
+            while (pl.wr < 4)
+            {
+                const int wp = 4 / pl.wr;
+                if ((size_t)32 * wp * (rank + 16 / elem) * elem <= 140 * 1024)
+                    break;
+                pl.wr *= 2;
+            }
+            const int pt = 32 * (4 / pl.wr);
+            pl.row_blocks = ceil_div(R, 16 * pl.wr);
+            int nsplit = ceil_div(LAT_TARGET, pl.row_blocks * n);
+            const int most = ceil_div(max_len, pt);
+            nsplit = nsplit < most ? nsplit : most;
+            pl.chunk = round_up(ceil_div(max_len, nsplit), pt);
+            pl.nsplit = ceil_div(max_len, pl.chunk);
+            return pl;
+        }
+    } // namespace
+} // namespace llamql
+
+using namespace llamql;
+
+extern "C" bool llam_seq_latent_append(const float *d_x, int ldx, const float *d_norm, float eps, int k_real,
+                                       const int32_t *d_row_slot, const int32_t *d_row_pos, void *d_cache, int M,
+                                       int rank, int cap, int dtype, int device_id, void *stream)
+{
+    static const char *fn = "llam_seq_latent_append";
+    if (M < 0 || rank < 1 || cap < 1 || k_real < 1 || k_real > rank || ldx < rank)
+        return fail(fn, "bad size (M=%d rank=%d cap=%d)", M, rank, cap);
+    if (M == 0)
+        return true;
+    if (!d_x || !d_norm || !d_row_slot || !d_row_pos || !d_cache)
+        return fail(fn, "null pointer");
+    if ((rank % PAD) != 0 || (ldx % 4) != 0 || !aligned16(d_x) || !aligned16(d_norm) || !aligned16(d_cache))
+        return fail(fn, "misaligned rows");
+    if (!set_device(fn, device_id))
+        return false;
+    if (dtype == LLAM_SEQ_F32)
+        hipLaunchKernelGGL(latent_append_kernel<float>, dim3(M), dim3(256), 0, as_stream(stream), d_x, ldx, d_norm, eps,
+                           k_real, d_row_slot, d_row_pos, static_cast<float *>(d_cache), rank, cap);
+    else
+        hipLaunchKernelGGL(latent_append_kernel<bf16>, dim3(M), dim3(256), 0, as_stream(stream), d_x, ldx, d_norm, eps,
+                           k_real, d_row_slot, d_row_pos, static_cast<bf16 *>(d_cache), rank, cap);
+    return launched(fn);
+}
+
+extern "C" size_t llam_seq_latent_scratch_floats(int max_rows, int slots, int heads, int rank, int cap)
+{
+    if (max_rows < 1 || slots < 1 || heads < 1 || rank < 1 || cap < 1)
+        return 0;
+    // rows that are split: fewer than LAT_TARGET workgroups of at most 64 rows, at most about
+    // 2 LAT_TARGET of them after the split; every entry of a call takes at least one row group
+    return ((size_t)2 * LAT_TARGET + slots) * 64 * ((size_t)rank + 2);
+}
+
+extern "C" bool llam_seq_latent_attention(const void *d_q, const void *d_cache, const llam_seq_entries *e, int first,
+                                          int n, int max_ntok, int max_len, int heads, int rank, int cap, float scale,
+                                          void *d_o, float *d_scratch, size_t scratch_floats, int dtype, int device_id,
+                                          void *stream)
+{
+    static const char *fn = "llam_seq_latent_attention";
+    if (n < 0 || first < 0 || heads < 1 || rank < 1 || cap < 1 || max_ntok < 1 || max_len < 1 || max_len > cap)
+        return fail(fn, "bad size (n=%d heads=%d rank=%d cap=%d max_ntok=%d max_len=%d)", n, heads, rank, cap, max_ntok, max_len);
+    if (n == 0)
+        return true;
+    if (!d_q || !d_cache || !e || !e->d_row0 || !e->d_ntok || !e->d_slot || !e->d_pos || !d_o || !d_scratch)
+        return fail(fn, "null pointer");
+    if ((rank % PAD) != 0 || !aligned16(d_q) || !aligned16(d_cache) || !aligned16(d_o) || !aligned16(d_scratch))
+        return fail(fn, "rank=%d must be a multiple of %d, rows 16-byte aligned", rank, PAD);
+    if (dtype != LLAM_SEQ_BF16 && dtype != LLAM_SEQ_F32)
+        return fail(fn, "dtype %d", dtype);
+    const LatentPlan pl = latent_plan(n, max_ntok, max_len, heads, rank, dtype == LLAM_SEQ_F32 ? 4 : 2);
+    LatentArgs p{};
+    p.q = d_q, p.cache = d_cache, p.row0 = e->d_row0, p.ntok = e->d_ntok, p.slot = e->d_slot, p.pos = e->d_pos;
+    p.first = first, p.heads = heads, p.rank = rank, p.cap = cap, p.chunk = pl.chunk, p.nsplit = pl.nsplit;
+    p.scale = scale, p.o = d_o, p.slices = 1;
+    p.rcap = max_ntok * heads;
+    const size_t parts = (size_t)n * pl.nsplit * p.rcap;
+    if (pl.nsplit > 1 && parts * ((size_t)rank + 2) > scratch_floats)
+        return fail(fn, "scratch too small");
+    p.part_o = d_scratch, p.part_ml = d_scratch + parts * rank;
+    if (n > 65535 || pl.nsplit > 65535)
+        return fail(fn, "too many entries");
+    if (!set_device(fn, device_id))
+        return false;
+    hipStream_t st = as_stream(stream);
+    bool ok;
+    if (dtype == LLAM_SEQ_F32)
+    {
+        if (rank <= 128)
+            ok = latent_rows<float, 8, true>(fn, p, pl.wr, pl.row_blocks, n, st);
+        else
+        {
+            p.slices = ceil_div(rank, 256);
+            ok = latent_rows<float, 16, false>(fn, p, pl.wr, pl.row_blocks, n, st);
+        }
+    }
+    else if (rank <= 128)
+        ok = latent_rows<bf16, 8, true>(fn, p, pl.wr, pl.row_blocks, n, st);
+    else if (rank <= 256)
+        ok = latent_rows<bf16, 16, true>(fn, p, pl.wr, pl.row_blocks, n, st);
+    else if (rank <= 512)
+        ok = latent_rows<bf16, 32, true>(fn, p, pl.wr, pl.row_blocks, n, st);
+    else
+    {
+        p.slices = ceil_div(rank, 256);
+        ok = latent_rows<bf16, 16, false>(fn, p, pl.wr, pl.row_blocks, n, st);
+    }
+    if (!ok || pl.nsplit == 1)
+        return ok;
+    if (dtype == LLAM_SEQ_F32)
+        hipLaunchKernelGGL(latent_merge_kernel<float>, dim3(p.rcap, n), dim3(LAT_MERGE_THREADS), 0, st, p);
+    else
+        hipLaunchKernelGGL(latent_merge_kernel<bf16>, dim3(p.rcap, n), dim3(LAT_MERGE_THREADS), 0, st, p);
+    return launched(fn);
+}
