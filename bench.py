@@ -369,6 +369,106 @@ def bench_decode(args, torch, capi, synth, dev):
     return out
 
 
+SEQUENCE_SIZES = {
+    # width, dense ff, experts (count, top, ff, shared ff), latent (heads, dim, vdim, q_rank, kv_rank), memory (heads, dim, vdim), and the
+    # quantized dense model of the same width, feed-forward width and number of layers
+    "2048": dict(width=2048, ff=8192, moe=(64, 6, 1408, 2816), latent=(16, 128, 128, 768, 512), memory=(4, 256, 512),
+                 dense=dict(hidden=2048, n_heads=32, n_kv=4, ffn=8192)),
+    "5120": dict(width=5120, ff=25600, moe=(64, 6, 1536, 3072), latent=(64, 128, 128, 1536, 512), memory=(8, 256, 512),
+                 dense=dict(hidden=5120, n_heads=64, n_kv=8, ffn=25600)),
+}
+
+
+def bench_sequence(args, torch, capi, synth, dev):
+    """Sequence model of four layers (memory + gated, latent attention + experts, memory + experts, latent
+    attention on the second layer's cache + gated) over random bf16 weights: prefill of a 2048-token portion and greedy
+    decoding at the given context, beside the quantized dense decoder of the same width, feed-forward width, depth
+    and vocabulary (whose step has no prefill: its prompts run token by token)."""
+    from llaminar_amd import sequence as sq
+    from llaminar_amd.decoder import DenseDecoder, Shape
+
+    def layer(z, mixer, ffn, kv_from=-1):
+        w = sq.Layer(mixer=mixer, kv_from=kv_from, ffn=ffn)
+        if mixer == sq.MIXER_LATENT_ATTENTION:
+            w.heads, w.dim, w.vdim, w.q_rank, w.kv_rank = z["latent"]
+        else:
+            w.heads, w.dim, w.vdim = z["memory"]
+        if ffn == sq.FFN_GATED:
+            w.ff = z["ff"]
+        else:
+            w.experts, w.top, w.ff, w.shared_ff = z["moe"]
+        return w
+
+    vocab, ctx, B, portion = 32768, args.context, args.batch, 2048
+    steps, rows = max(args.steps, 20), []
+    for name in args.sizes.split(","):
+        z = SEQUENCE_SIZES[name]
+        LAT, MEM, GATED, EXPERTS = sq.MIXER_LATENT_ATTENTION, sq.MIXER_MATRIX_MEMORY, sq.FFN_GATED, sq.FFN_EXPERTS
+        layers = [layer(z, MEM, GATED), layer(z, LAT, EXPERTS), layer(z, MEM, EXPERTS), layer(z, LAT, GATED, kv_from=1)]
+        cap = ctx + steps + args.warmup + 16
+        model = synth.sequence_model_torch(layers, z["width"], vocab, dev, slots=B, cap=cap, max_rows=portion)
+        ids = torch.randint(0, vocab, (portion,), generator=torch.Generator().manual_seed(1)).numpy()
+        for slot in range(B):   # the context every decode step finds
+            for at in range(0, ctx, portion):
+                model.forward([(slot, at, ids[:min(portion, ctx - at)])])
+        row = {"width": z["width"], "batch": B, "context": ctx, "layers": 4}
+        if args.phase in ("prefill", "both"):
+            reps = max(3, min(20, args.steps // 10))
+            for at, key in ((0, "prefill_ms_first_portion"), (ctx - portion, "prefill_ms_last_portion")):
+                if at < 0:
+                    continue
+                t0 = time.perf_counter()
+                for _ in range(reps):
+                    model.forward([(0, at, ids)], [portion - 1], best=True)
+                row[key] = round((time.perf_counter() - t0) * 1e3 / reps, 3)
+            row["prefill_tokens_per_s"] = round(portion * 1e3 / row["prefill_ms_first_portion"], 1)
+        if args.phase in ("decode", "both"):
+            pos, slots, tok = [ctx] * B, list(range(B)), [1] * B
+            model.decode(slots, pos, tok, max(args.warmup, 2))
+            model.decode(slots, pos, tok, steps)
+            row["decode_ms"] = round(model.last_decode_ms / steps, 4)
+            row["decode_tokens_per_s"] = round(B * 1e3 / row["decode_ms"], 1)
+            row["weight_bytes_batch1"] = sum(model.weight_bytes)
+            row["state_bytes_per_step"] = B * (2 * sum(w.heads * sq.P(w.dim) * (sq.P(w.vdim) + 16) * 8 for w in layers[:1]) +
+                                               2 * ctx * layers[1].kv_rank * 2)
+            row["hbm_frac_batch1_bytes"] = round((row["weight_bytes_batch1"] + row["state_bytes_per_step"]) / (row["decode_ms"] * 1e-3) / 8e12, 4)
+        model.close()
+        del model
+        torch.cuda.empty_cache()
+        if args.phase in ("decode", "both") and not args.no_decode:
+            shape = Shape(n_layers=4, vocab=vocab, **z["dense"])
+            dec = DenseDecoder(shape, B, (cap + 31) // 32 * 32, dev, seed=11)
+            dec.set_state([1] * B, [ctx - 1] * B)
+            stream = torch.cuda.Stream()
+            with torch.cuda.stream(stream):
+                dec.step(stream)
+                stream.synchronize()
+                graph = torch.cuda.CUDAGraph()
+                with torch.cuda.graph(graph, stream=stream):
+                    dec.step(stream)
+                graph.replay()
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                for _ in range(steps):
+                    graph.replay()
+                torch.cuda.synchronize()
+                ms = (time.perf_counter() - t0) * 1e3 / steps
+            kv = 4 * B * 2 * shape.n_kv * ctx * shape.head_dim * 2
+            row["dense_q4k"] = {"decode_ms": round(ms, 4), "decode_tokens_per_s": round(B * 1e3 / ms, 1),
+                                "bytes_per_step": shape.weight_bytes_per_token() + kv,
+                                "hbm_frac": round((shape.weight_bytes_per_token() + kv) / (ms * 1e-3) / 8e12, 4)}
+            dec.close()
+            del dec
+            torch.cuda.empty_cache()
+        rows.append(row)
+    first = rows[0]
+    if args.phase == "prefill":
+        metric, value, ms = "sequence-model prefill tokens/s", first["prefill_tokens_per_s"], first["prefill_ms_first_portion"]
+    else:
+        metric, value, ms = "sequence-model decode tokens/s (batch %d)" % B, first["decode_tokens_per_s"], first["decode_ms"]
+    return _common(args, metric, value, "tokens/s", ms, "bf16", {"workload": bench_sequence.__doc__.strip(), "sizes": rows}, None)
+
+
 def bench_read_order(args, torch, capi, synth, dev):
     """What the order of a GEMV's reads is worth on its own: read-only kernels over 25600 x 5120 Q4_K-sized buffers
     (73.7 MB each, eight rotated so nothing is served from a previous launch), no arithmetic."""
@@ -419,7 +519,7 @@ def bench_read_order(args, torch, capi, synth, dev):
 
 
 OTHER_WORKLOADS = {"gemm": bench_gemm, "moe": bench_moe, "gemv": bench_gemv, "decode": bench_decode,
-                   "read-order": bench_read_order}
+                   "read-order": bench_read_order, "sequence": bench_sequence}
 
 
 def parse():
@@ -429,10 +529,14 @@ def parse():
     ap.add_argument("--warmup", type=int, default=20)
     ap.add_argument("--moe-path", choices=["auto", "slots", "grouped-gate-up", "grouped"], default="auto",
                     help="moe workload: per-slot launches, or tokens grouped by expert (gate/up only, or down as well)")
-    ap.add_argument("--workload", choices=["layer", "gemm", "moe", "gemv", "decode", "read-order"], default="layer",
+    ap.add_argument("--workload", choices=["layer", "gemm", "moe", "gemv", "decode", "read-order", "sequence"], default="layer",
                     help="layer: the headline decode-layer step (default); gemm: prefill int8 GEMM 512x25600x5120 Q4_K; "
                          "moe: 256-expert top-8 IQ3_S expert FFN decode; gemv: single GEMVs of every format and layer shape; "
-                         "read-order: read-only probes of the GEMV's load stream in several orders")
+                         "read-order: read-only probes of the GEMV's load stream in several orders; "
+                         "sequence: prefill and decoding of a sequence model (latent attention, matrix memory, experts; bf16 weights) "
+                         "beside the quantized dense decoder of the same width")
+    ap.add_argument("--sizes", default="2048,5120", help="sequence workload: widths, with commas between them")
+    ap.add_argument("--phase", choices=["prefill", "decode", "both"], default="both", help="sequence workload: what is timed")
     ap.add_argument("--batch", type=int, default=1, help="activation rows / tokens per step")
     ap.add_argument("--layers", type=int, default=4, help="distinct weight sets rotated through")
     ap.add_argument("--no-graph", action="store_true", help="launch eagerly instead of replaying HIP graphs")

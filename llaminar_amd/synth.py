@@ -54,3 +54,84 @@ def activations_numpy(M: int, K: int, seed: int) -> np.ndarray:
 def gemv_bytes(fmt: int, N: int, K: int, M: int = 1) -> int:
     """Algorithmic bytes of one GEMV: weights + Q8_1 activations + fp32 outputs."""
     return N * (K // 256) * BLOCK_BYTES[fmt] + M * (K // 32) * 36 + M * N * 4
+
+
+def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap: int, max_rows: int = 2048,
+                         dtype: str = "bfloat16", eps: float = 1e-5, seed: int = 0):
+    """A sequence.SequenceModel of random bf16 weights made on the device (matrices too big to build on the host
+    every run).  ``layers``: sequence.Layer descriptions with sizes only; every tensor is filled in here, N(0, 1/in)
+    (random weights need no particular order of tiles).  The tensors live as long as the model."""
+    import ctypes
+
+    import torch
+
+    from . import sequence as sq
+
+    g = torch.Generator(device=device)
+    g.manual_seed(seed)
+    P = sq.P
+    model = sq.SequenceModel.__new__(sq.SequenceModel)
+    model.L, model.keep = sq.load(), []
+    model.width, model.vocab, model.slots, model.cap, model.max_rows, model.n_layers = width, vocab, slots, cap, max_rows, len(layers)
+    model.weight_bytes = []   # per layer: bf16 bytes a decode step reads at batch 1
+    model.h = model.L.llam_seqm_create(ctypes.byref(sq.Config(width, vocab, len(layers), slots, cap, max_rows, sq.DTYPES[dtype],
+                                                              eps, device.index or 0)))
+    if not model.h:
+        raise sq.SequenceError(model._error())
+
+    def matrix(rows, columns, count=1):
+        t = torch.empty(count * sq.pad_to(rows, 16) * P(columns), dtype=torch.bfloat16, device=device)
+        t.normal_(0.0, columns ** -0.5, generator=g)
+        model.keep.append(t)
+        return t.data_ptr(), t.numel() * 2
+
+    def vector(n, value=1.0):
+        t = torch.full((n,), value, device=device)
+        model.keep.append(t)
+        return t.data_ptr()
+
+    for n, w in enumerate(layers):
+        H, d, v, wp, read = w.heads, P(w.dim), P(w.vdim), P(width), 0
+        w.norm1 = vector(wp)
+        w.w_out, b = matrix(wp, H * v)
+        read += b
+        if w.mixer == sq.MIXER_LATENT_ATTENTION:
+            own = w.kv_from < 0
+            w.w_in, b1 = matrix(P(w.q_rank) + (P(w.kv_rank) if own else 0), wp)
+            w.w_uq, b2 = matrix(H * d, w.q_rank)
+            w.w_uk_t, b3 = matrix(H * P(w.kv_rank), d)
+            w.w_uv, b4 = matrix(H * v, w.kv_rank)
+            read += b1 + b2 + b3 + b4
+            w.q_norm, w.kv_norm = vector(P(w.q_rank)), vector(P(w.kv_rank))
+            w.scale = w.scale or w.dim ** -0.5
+        else:
+            w.w_in, b = matrix(2 * H * (d + v) + 2 * H, wp)
+            read += b
+            w.gate_bias, w.head_norm = vector(2 * H, 2.0), vector(H * v)
+            w.gate_cap, w.scale = w.gate_cap or 15.0, w.dim ** -0.5
+        if w.ffn:
+            w.norm2 = vector(wp)
+        if w.ffn == sq.FFN_GATED:
+            w.w_up, b1 = matrix(2 * P(w.ff), wp)
+            w.w_down, b2 = matrix(wp, P(w.ff))
+            read += b1 + b2
+        elif w.ffn == sq.FFN_EXPERTS:
+            w.w_up, b1 = matrix(P(w.ff), wp, w.experts)
+            w.w_down, b2 = matrix(wp, P(w.ff), w.experts)
+            rows = w.experts + (1 if w.shared_ff else 0)
+            w.w_router, b3 = matrix(rows, wp)
+            w.router_bias = vector(sq.pad_to(rows, 16), 0.0)
+            read += (b1 + b2) * w.top // w.experts + b3
+            if w.shared_ff:
+                w.w_shared_up, b4 = matrix(P(w.shared_ff), wp)
+                w.w_shared_down, b5 = matrix(wp, P(w.shared_ff))
+                read += b4 + b5
+        model.weight_bytes.append(read)
+        model._check(model.L.llam_seqm_set_layer(model.h, n, ctypes.byref(w)))
+    embed = torch.randn(vocab, width, device=device, generator=g).to(torch.bfloat16)
+    model.keep.append(embed)
+    head, b = matrix(vocab, P(width))
+    model.weight_bytes.append(b)
+    torch.cuda.synchronize()
+    model._check(model.L.llam_seqm_set_globals(model.h, ctypes.byref(sq.Globals(embed.data_ptr(), vector(P(width)), head))))
+    return model

@@ -48,7 +48,7 @@ def check(got, want, dtype, f32=2e-5, bf16=0.02, note=""):
     if dtype == "float32":
         # where a memory's output nearly cancels, the norm behind it magnifies the last bits (weights changed by half
         # a 32-bit rounding move such rows by 1e-5): a few rows may be further off, a wrong one is off by 1e-2
-        ok = np.median(e) < f32 / 5 and np.mean(e > f32) <= 0.03 and e.max() < 30 * f32
+        ok = np.median(e) < f32 / 5 and np.mean(e > f32) <= 0.05 and e.max() < 30 * f32
         assert ok, (note, int(e.argmax()), float(e.max()), float(np.median(e)))
     else:
         # a router may choose otherwise where two logits are within a bfloat16 rounding: a few rows
