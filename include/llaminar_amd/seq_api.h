@@ -117,7 +117,7 @@ typedef struct
     int heads, dim, vdim, vdim_real;
     float q_scale, gate_cap, eps;
 } llam_seq_memory_args;
-size_t llam_seq_memory_scratch_bytes(int max_rows, int heads, int vdim);
+size_t llam_seq_memory_scratch_bytes(int max_rows, int heads, int dim, int vdim);
 /* one token per entry, entries first .. first + n - 1 */
 bool llam_seq_memory_decode(const llam_seq_memory_args *a, const llam_seq_entries *e, int first, int n,
                             void *d_scratch, size_t scratch_bytes, int dtype, int device_id, void *stream);

@@ -3,19 +3,28 @@
 // Queries arrive in latent space (q . W_uk, one vector of `rank` per head), so all heads of a
 // token share every cache row: a query row is a (token, head) pair, R = tokens * heads rows per
 // entry, all against the same keys.  A workgroup takes 16 WR rows and a stretch of the sequence,
-// walks it 32 WP positions at a time (WR * WP = 4 wavefronts), the cache rows staged once in LDS:
-//   scores  S[row][p] = sum_d q[row][d] c[p][d]   second operand: c rows as they lie
-//   output  O[row][d] = sum_p w[row][p] c[p][d]   second operand: c columns (transposing LDS read)
-// with a running maximum per row.  Softmax in 32-bit; for bf16 the weights enter the second
-// product as two bf16 pieces.  With WP > 1 the wavefronts of a row group split the positions and
-// merge through LDS; with several stretches per row group a second kernel merges those.
+// and walks it 32 WP positions at a time (WR * WP = 4 groups of two wavefronts), the cache rows
+// staged once in LDS:
+//   scores  S[row][p] = sum_d q[row][d] c[p][d]   second operand: c rows as they lie; each wavefront
+//                                                  of a pair takes 16 of the group's 32 positions
+//   output  O[row][d] = sum_p w[row][p] c[p][d]   second operand: c columns (transposing LDS read);
+//                                                  each takes half of the columns
+// In between the scores pass through LDS, where both read them as first operand of the output
+// product and keep the running maximum and sum of their rows.  Softmax in 32-bit; for bf16 the
+// weights enter the product as two bf16 pieces.  With WP > 1 the groups of a row block split the
+// positions and merge through LDS; with several stretches per row block a second kernel merges those.
 #include "seq_common.h"
 #include "llaminar_amd/seq_api.h"
 
 namespace llamql
 {
-    constexpr int LAT_THREADS = 256;
-    constexpr int LAT_TARGET = 512; // workgroups aimed at before rows are no longer split
+    constexpr int LAT_THREADS = 512;
+    constexpr int LAT_TARGET = 256; // workgroups aimed at before rows are no longer split
+    constexpr int LAT_MIN_STRETCH = 64; // positions: shorter stretches cost more in partial results than they gain
+
+    constexpr int LAT_PAD = 32;         // bytes between staged rows: both kinds of LDS read spread over the banks
+
+    __device__ __forceinline__ float fast_exp(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
 
     struct LatentArgs
     {
@@ -28,23 +37,26 @@ namespace llamql
         float *part_o, *part_ml;
     };
 
-    // NOUT: 16-column output tiles of a wavefront.  QREG: the query rows stay in registers (rank <= 16 NOUT);
-    // otherwise they are read again for every stretch and blockIdx.z also counts output slices.
+    // NOUT: 16-column output tiles of a row block, half of them per wavefront.  QREG: the query rows stay in
+    // registers (rank <= 16 NOUT); otherwise they are read again for every turn and blockIdx.z also counts
+    // slices of the output.
     template <typename T, int NOUT, bool QREG, int WR>
     __global__ void __launch_bounds__(LAT_THREADS)
         latent_attention_kernel(LatentArgs p)
     {
         using O = Operand<T>;
         using V = typename O::V;
+        typedef T t4 __attribute__((ext_vector_type(4)));
         constexpr int WP = 4 / WR, PT = 32 * WP;
-        constexpr int LPAD = 16 / sizeof(T);
+        constexpr int LPAD = LAT_PAD / sizeof(T);
         constexpr int PW = sizeof(T) == 2 ? 2 : 1; // pieces of a softmax weight
         constexpr int SLD = 36;
+        constexpr int NT = NOUT / 2;               // output tiles of a wavefront
         extern __shared__ __attribute__((aligned(16))) char smem[];
-        __shared__ __attribute__((aligned(16))) float s_p[4][16 * SLD];
+        __shared__ __attribute__((aligned(16))) float s_s[4][16 * SLD];
         const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
         const int c = lane & 15, g = lane >> 4;
-        const int wr = wave % WR, wp = wave / WR;
+        const int half = wave & 1, group = wave >> 1, wr = group % WR, wp = group / WR;
         const int ei = QREG ? blockIdx.z : blockIdx.z / p.slices;
         const int slice = QREG ? 0 : blockIdx.z % p.slices;
         const int e = p.first + ei, split = blockIdx.y;
@@ -53,7 +65,7 @@ namespace llamql
         if (rb >= R)
             return;
         const int last_row = rb + 16 * WR - 1 < R ? rb + 16 * WR - 1 : R - 1;
-        const int kmax = pos0 + last_row / p.heads; // newest position any row of the group sees
+        const int kmax = pos0 + last_row / p.heads; // newest position any row of the block sees
         const int k0 = split * p.chunk;
         if (k0 > kmax || kmax >= p.cap)
             return;
@@ -61,8 +73,33 @@ namespace llamql
 
         const int ksteps = p.rank >> 5;
         const int ld = p.rank + LPAD;
-        T *tile = reinterpret_cast<T *>(smem);
         const T *cache = static_cast<const T *>(p.cache) + (size_t)p.slot[e] * p.cap * p.rank;
+
+        // The cache rows of a turn: TPR threads a row.  With two buffers the next turn's rows are requested
+        // before this turn's products and put down in the middle of them.
+        constexpr int TPR = LAT_THREADS / PT;
+        constexpr int LOADS = NOUT * (int)sizeof(T) >= TPR ? NOUT * (int)sizeof(T) / TPR : 1; // 16-byte pieces a thread, when QREG
+        constexpr bool AHEAD = QREG && WP == 1;
+        constexpr int BATCH = LOADS < 8 ? LOADS : 8; // held at once
+        const int pieces = p.rank * (int)sizeof(T) / 16;
+        const int srow = threadIdx.x / TPR, sseg = threadIdx.x % TPR;
+        u32x4 held[QREG ? BATCH : 1];
+        auto request = [&](int p0, int i0) __attribute__((always_inline)) {
+            // rows past the end are masked; they only must be numbers
+            const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)(p0 + srow <= kmax ? p0 + srow : kmax) * p.rank) + sseg;
+#pragma unroll
+            for (int i = 0; i < BATCH; ++i)
+                held[i] = src[sseg + (i0 + i) * TPR < pieces ? (i0 + i) * TPR : 0];
+        };
+        auto put = [&](int buf, int i0) __attribute__((always_inline)) {
+            u32x4 *dst = reinterpret_cast<u32x4 *>(reinterpret_cast<T *>(smem) + (buf * PT + srow) * ld) + sseg;
+#pragma unroll
+            for (int i = 0; i < BATCH; ++i)
+                if (sseg + (i0 + i) * TPR < pieces)
+                    dst[(i0 + i) * TPR] = held[i];
+        };
+        if constexpr (AHEAD)
+            request(k0, 0);
 
         const int qrow = rb + wr * 16 + c < R ? rb + wr * 16 + c : R - 1;
         const T *q = static_cast<const T *>(p.q) + ((size_t)p.row0[e] * p.heads + qrow) * p.rank + 8 * g;
@@ -74,199 +111,241 @@ namespace llamql
                 if (ks < ksteps)
                     qreg[ks] = O::load(q + ks * 32);
         }
-        int limit[4]; // newest position of this lane's result rows 4 g + r
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-        {
-            const int row = rb + wr * 16 + 4 * g + r;
-            limit[r] = row < R ? pos0 + row / p.heads : -1;
-        }
-        const int out_tiles = (p.rank >> 4) - slice * NOUT < NOUT ? (p.rank >> 4) - slice * NOUT : NOUT;
+        const int limit = rb + wr * 16 + c < R ? pos0 + qrow / p.heads : -1; // newest position this lane's row c sees
+        const int tile0 = slice * NOUT + half * NT;                         // the wavefront's first output tile
+        const int out_tiles = (p.rank >> 4) - tile0 < NT ? (p.rank >> 4) - tile0 : NT;
 
-        float m[4], l[4];
-        f32x4 acc[NOUT];
+        float m = -INFINITY, l = 0.0f; // of row c; l: this lane's positions only
+        f32x4 acc[NT];
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-        {
-            m[r] = -INFINITY;
-            l[r] = 0.0f;
-        }
-#pragma unroll
-        for (int t = 0; t < NOUT; ++t)
+        for (int t = 0; t < NT; ++t)
             acc[t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-
-        const int pieces = p.rank * (int)sizeof(T) / 16;
+        int buf = 0;
+        if constexpr (AHEAD)
+        {
+            put(0, 0);
+            if (k0 + PT < k1)
+                request(k0 + PT, 0);
+        }
         for (int kt = k0; kt < k1; kt += PT)
         {
-            __syncthreads();
-            for (int r = threadIdx.x >> 3; r < PT; r += LAT_THREADS / 8)
+            if constexpr (!AHEAD)
             {
-                const int pos = kt + r <= kmax ? kt + r : kmax; // rows past the end are masked; they only must be numbers
-                const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)pos * p.rank);
-                u32x4 *dst = reinterpret_cast<u32x4 *>(tile + r * ld);
-                for (int i = threadIdx.x & 7; i < pieces; i += 8)
-                    dst[i] = src[i];
+                __syncthreads();
+                if constexpr (QREG)
+                {
+#pragma unroll
+                    for (int i = 0; i < LOADS; i += BATCH)
+                    {
+                        request(kt, i);
+                        put(0, i);
+                    }
+                }
+                else
+                {
+                    const int pos = kt + srow <= kmax ? kt + srow : kmax;
+                    const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)pos * p.rank);
+                    u32x4 *dst = reinterpret_cast<u32x4 *>(reinterpret_cast<T *>(smem) + srow * ld);
+                    for (int i = sseg; i < pieces; i += TPR)
+                        dst[i] = src[i];
+                }
             }
             __syncthreads();
 
-            const T *mine = tile + wp * 32 * ld;
+            const T *mine = reinterpret_cast<const T *>(smem) + (buf * PT + wp * 32) * ld;
+            const T *keys = mine + (16 * half + c) * ld + 8 * g;
             f32x4 s[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
             if (QREG)
             {
 #pragma unroll
                 for (int ks = 0; ks < NOUT / 2; ++ks)
                     if (ks < ksteps)
-                    {
-                        s[0] = O::mma(qreg[ks], O::load(mine + c * ld + ks * 32 + 8 * g), s[0]);
-                        s[1] = O::mma(qreg[ks], O::load(mine + (16 + c) * ld + ks * 32 + 8 * g), s[1]);
-                    }
+                        s[ks & 1] = O::mma(qreg[ks], O::load(keys + ks * 32), s[ks & 1]);
             }
             else
-                for (int ks = 0; ks < ksteps; ++ks)
+                for (int ks = 0; ks < ksteps; ks += 2) // (the rank is a multiple of 64)
                 {
-                    const V a = O::load(q + ks * 32);
-                    s[0] = O::mma(a, O::load(mine + c * ld + ks * 32 + 8 * g), s[0]);
-                    s[1] = O::mma(a, O::load(mine + (16 + c) * ld + ks * 32 + 8 * g), s[1]);
+                    s[0] = O::mma(O::load(q + ks * 32), O::load(keys + ks * 32), s[0]);
+                    s[1] = O::mma(O::load(q + ks * 32 + 32), O::load(keys + ks * 32 + 32), s[1]);
                 }
-            float alpha[4];
+            s[0] = s[0] + s[1];
 #pragma unroll
             for (int r = 0; r < 4; ++r)
+                s_s[group][(4 * g + r) * SLD + 16 * half + c] = s[0][r];
+            if constexpr (AHEAD)
             {
-                const int pa = kt + wp * 32 + c;
-                const float sa = pa <= limit[r] ? s[0][r] * p.scale : -INFINITY;
-                const float sb = pa + 16 <= limit[r] ? s[1][r] * p.scale : -INFINITY;
-                float mx = fmaxf(sa, sb);
-#pragma unroll
-                for (int off = 1; off < 16; off <<= 1)
-                    mx = fmaxf(mx, __shfl_xor(mx, off, 64));
-                const float mn = fmaxf(m[r], mx);
-                const float base = mn == -INFINITY ? 0.0f : mn;
-                alpha[r] = expf(m[r] - base);
-                m[r] = mn;
-                const float ea = expf(sa - base), eb = expf(sb - base);
-                l[r] = l[r] * alpha[r] + ea + eb;
-                s_p[wave][(4 * g + r) * SLD + c] = ea;
-                s_p[wave][(4 * g + r) * SLD + 16 + c] = eb;
-            }
-            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-            __builtin_amdgcn_wave_barrier();
-            __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-            V w[PW];
-            {
-                const f32x4 a = *reinterpret_cast<const f32x4 *>(&s_p[wave][c * SLD + 8 * g]);
-                const f32x4 b = *reinterpret_cast<const f32x4 *>(&s_p[wave][c * SLD + 8 * g + 4]);
-                split_pieces<T, PW>(__builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7), w);
-            }
-#pragma unroll
-            for (int t = 0; t < NOUT; ++t)
-                if (t < out_tiles)
+                if (kt + PT < k1)
                 {
-                    const V v = load_columns(mine + (slice * NOUT + t) * 16, ld, lane);
+                    put(buf ^ 1, 0);
+                    if (kt + 2 * PT < k1)
+                        request(kt + 2 * PT, 0);
+                }
+            }
+            __syncthreads();
+
+            // row c, positions 8 g .. 8 g + 7 of the group's 32
+            f32x8 w = Operand<float>::load(&s_s[group][c * SLD + 8 * g]);
+            float mx = m;
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+            {
+                w[j] = kt + wp * 32 + 8 * g + j <= limit ? w[j] * p.scale : -INFINITY;
+                mx = fmaxf(mx, w[j]);
+            }
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            const float base = mx == -INFINITY ? 0.0f : mx;
+            const float alpha = fast_exp(m - base);
+            const bool moved = mx != m;
+            m = mx;
+            l *= alpha;
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+            {
+                w[j] = fast_exp(w[j] - base);
+                l += w[j];
+            }
+            V wv[PW];
+            split_pieces<T, PW>(w, wv);
+            if (__any(moved)) // most turns move no maximum
+            {
+                float a[4];
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    a[r] = __shfl(alpha, 4 * g + r, 64);
+#pragma unroll
+                for (int t = 0; t < NT; ++t)
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
-                        acc[t][r] *= alpha[r];
+                        acc[t][r] *= a[r];
+            }
+            constexpr int VG = sizeof(T) == 2 ? 4 : 2; // independent products in a row (NT is a multiple)
+#pragma unroll
+            for (int t = 0; t < NT; t += VG)
+                if (t < out_tiles)
+                {
+                    V v[VG];
+#pragma unroll
+                    for (int k = 0; k < VG; ++k) // (a tile past the rank: the first one again, its result is not used)
+                        v[k] = load_columns(mine + (tile0 + (t + k < out_tiles ? t + k : 0)) * 16, ld, lane);
 #pragma unroll
                     for (int i = 0; i < PW; ++i)
-                        acc[t] = O::mma(w[i], v, acc[t]);
+#pragma unroll
+                        for (int k = 0; k < VG; ++k)
+                            acc[t + k] = O::mma(wv[i], v[k], acc[t + k]);
                 }
+            if constexpr (AHEAD)
+                buf ^= 1;
         }
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-#pragma unroll
-            for (int off = 1; off < 16; off <<= 1)
-                l[r] += __shfl_xor(l[r], off, 64);
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
 
         if (WP > 1)
         {
-            // merge the wavefronts of each row group: [wave][16 rows][16 NOUT columns], then (m, l)
+            // merge the groups of each row block: [group][16 rows][16 NOUT columns], then (m, l) of their rows
             __syncthreads();
             float *s_o = reinterpret_cast<float *>(smem);
-            float *s_ml = &s_p[0][0];
+            float *s_ml = &s_s[0][0];
             constexpr int OLD = NOUT * 16 + 4;
 #pragma unroll
-            for (int t = 0; t < NOUT; ++t)
+            for (int t = 0; t < NT; ++t)
                 if (t < out_tiles)
                 {
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
-                        s_o[(wave * 16 + 4 * g + r) * OLD + t * 16 + c] = acc[t][r];
+                        s_o[(group * 16 + 4 * g + r) * OLD + (half * NT + t) * 16 + c] = acc[t][r];
                 }
-            if (c == 0)
+            if (half == 0 && g == 0)
             {
-#pragma unroll
-                for (int r = 0; r < 4; ++r)
-                {
-                    s_ml[(wave * 16 + 4 * g + r) * 2] = m[r];
-                    s_ml[(wave * 16 + 4 * g + r) * 2 + 1] = l[r];
-                }
+                s_ml[(group * 16 + c) * 2] = m;
+                s_ml[(group * 16 + c) * 2 + 1] = l;
             }
             __syncthreads();
-            for (int i = threadIdx.x; i < WR * 16 * out_tiles * 16; i += LAT_THREADS)
+            // per row: the groups' factors e^(m_w - M) (over the sum, when the result is final)
+            float *s_f = s_ml + 128;
+            if (threadIdx.x < WR * 16)
             {
-                const int row = i / (out_tiles * 16), d = i - row * (out_tiles * 16); // row of the group
-                if (rb + row >= R)
-                    continue;
+                const int row = threadIdx.x;
                 float M = -INFINITY;
 #pragma unroll
                 for (int w = 0; w < WP; ++w)
-                    M = fmaxf(M, s_ml[((w * WR * 16) + row) * 2]);
+                    M = fmaxf(M, s_ml[(w * WR * 16 + row) * 2]);
                 const float base = M == -INFINITY ? 0.0f : M;
-                float L = 0.0f, y = 0.0f;
+                float L = 0.0f, f[WP];
 #pragma unroll
                 for (int w = 0; w < WP; ++w)
                 {
-                    const float f = expf(s_ml[((w * WR * 16) + row) * 2] - base);
-                    L += f * s_ml[((w * WR * 16) + row) * 2 + 1];
-                    y += f * s_o[(w * WR * 16 + row) * OLD + d];
+                    f[w] = fast_exp(s_ml[(w * WR * 16 + row) * 2] - base);
+                    L += f[w] * s_ml[(w * WR * 16 + row) * 2 + 1];
                 }
-                const int col = slice * NOUT * 16 + d;
-                if (p.nsplit == 1)
-                    static_cast<T *>(p.o)[((size_t)p.row0[e] * p.heads + rb + row) * p.rank + col] = (T)(y / L);
-                else
+                const float inv = p.nsplit == 1 ? 1.0f / L : 1.0f;
+#pragma unroll
+                for (int w = 0; w < WP; ++w)
+                    s_f[w * WR * 16 + row] = f[w] * inv;
+                if (p.nsplit > 1 && slice == 0 && rb + row < R)
                 {
                     const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + rb + row;
-                    p.part_o[at * p.rank + col] = y;
-                    if (d == 0 && slice == 0)
-                    {
-                        p.part_ml[at * 2] = M;
-                        p.part_ml[at * 2 + 1] = L;
-                    }
+                    p.part_ml[at * 2] = M;
+                    p.part_ml[at * 2 + 1] = L;
                 }
             }
+            __syncthreads();
+            // a wavefront takes every eighth row
+            const int columns = p.rank - slice * NOUT * 16 < NOUT * 16 ? p.rank - slice * NOUT * 16 : NOUT * 16;
+            for (int row = wave; row < WR * 16 && rb + row < R; row += LAT_THREADS / 64)
+                for (int d = lane * 4; d < columns; d += 256)
+                {
+                    f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+                    for (int w = 0; w < WP; ++w)
+                        y = y + *reinterpret_cast<const f32x4 *>(s_o + (w * WR * 16 + row) * OLD + d) * s_f[w * WR * 16 + row];
+                    const int col = slice * NOUT * 16 + d;
+                    if (p.nsplit == 1)
+                        *reinterpret_cast<t4 *>(static_cast<T *>(p.o) + ((size_t)p.row0[e] * p.heads + rb + row) * p.rank + col) =
+                            __builtin_convertvector(y, t4);
+                    else
+                        *reinterpret_cast<f32x4 *>(p.part_o + (((size_t)ei * p.nsplit + split) * p.rcap + rb + row) * p.rank + col) = y;
+                }
             return;
         }
 #pragma unroll
         for (int r = 0; r < 4; ++r)
         {
             const int row = rb + wr * 16 + 4 * g + r;
+            const float inv = 1.0f / __shfl(l, 4 * g + r, 64);
             if (row >= R)
                 continue;
             const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + row;
-            const float inv = 1.0f / l[r];
 #pragma unroll
-            for (int t = 0; t < NOUT; ++t)
+            for (int t = 0; t < NT; ++t)
                 if (t < out_tiles)
                 {
-                    const int col = (slice * NOUT + t) * 16 + c;
+                    const int col = (tile0 + t) * 16 + c;
                     if (p.nsplit == 1)
                         static_cast<T *>(p.o)[((size_t)p.row0[e] * p.heads + row) * p.rank + col] = (T)(acc[t][r] * inv);
                     else
                         p.part_o[at * p.rank + col] = acc[t][r];
                 }
-            if (p.nsplit > 1 && c == 0 && slice == 0)
-            {
-                p.part_ml[at * 2] = m[r];
-                p.part_ml[at * 2 + 1] = l[r];
-            }
+        }
+        if (p.nsplit > 1 && half == 0 && g == 0 && slice == 0 && rb + wr * 16 + c < R)
+        {
+            const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + rb + wr * 16 + c;
+            p.part_ml[at * 2] = m;
+            p.part_ml[at * 2 + 1] = l;
         }
     }
 
-    // one workgroup per query row: o = sum_s o_s e^(m_s - M) / sum_s l_s e^(m_s - M)
-    constexpr int LAT_MERGE_THREADS = 128;
+    // o = sum_s o_s e^(m_s - M) / sum_s l_s e^(m_s - M): one workgroup per query row and 128 columns, eight groups
+    // of 32 threads dealing the stretches among themselves
+    constexpr int LAT_MERGE_COLS = 128;
     template <typename T>
-    __global__ void __launch_bounds__(LAT_MERGE_THREADS)
+    __global__ void __launch_bounds__(256)
         latent_merge_kernel(LatentArgs p)
     {
+        typedef T t4 __attribute__((ext_vector_type(4)));
+        __shared__ __attribute__((aligned(16))) float s_y[8][LAT_MERGE_COLS];
+        __shared__ float s_w[LAT_TARGET + 256];
+        __shared__ float s_red[4];
         const int ei = blockIdx.y, e = p.first + ei, row = blockIdx.x;
         if (row >= p.ntok[e] * p.heads)
             return;
@@ -275,22 +354,40 @@ namespace llamql
             return;
         const int used = limit / p.chunk + 1;
         const size_t at = (size_t)ei * p.nsplit * p.rcap + row;
+        const int group = threadIdx.x >> 5, d = blockIdx.z * LAT_MERGE_COLS + (threadIdx.x & 31) * 4;
         float M = -INFINITY;
-        for (int s = 0; s < used; ++s)
+        for (int s = threadIdx.x; s < used; s += 256)
             M = fmaxf(M, p.part_ml[(at + (size_t)s * p.rcap) * 2]);
-        for (int d = threadIdx.x * 4; d < p.rank; d += LAT_MERGE_THREADS * 4)
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1)
+            M = fmaxf(M, __shfl_xor(M, off, 64));
+        if ((threadIdx.x & 63) == 0)
+            s_red[threadIdx.x >> 6] = M;
+        __syncthreads();
+        M = fmaxf(fmaxf(s_red[0], s_red[1]), fmaxf(s_red[2], s_red[3]));
+        float L = 0.0f;
+        for (int s = threadIdx.x; s < used; s += 256)
         {
-            float L = 0.0f;
-            f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll 4
-            for (int s = 0; s < used; ++s)
-            {
-                const size_t k = at + (size_t)s * p.rcap;
-                const float f = expf(p.part_ml[k * 2] - M);
-                L += f * p.part_ml[k * 2 + 1];
-                y = y + *reinterpret_cast<const f32x4 *>(p.part_o + k * p.rank + d) * f;
-            }
-            typedef T t4 __attribute__((ext_vector_type(4)));
+            const size_t k = (at + (size_t)s * p.rcap) * 2;
+            const float f = expf(p.part_ml[k] - M);
+            s_w[s] = f;
+            L += f * p.part_ml[k + 1];
+        }
+        L = block_sum<256>(L, s_red);
+        f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
+        if (d < p.rank)
+        {
+#pragma unroll 8
+            for (int s = group; s < used; s += 8)
+                y = y + *reinterpret_cast<const f32x4 *>(p.part_o + (at + (size_t)s * p.rcap) * p.rank + d) * s_w[s];
+        }
+        *reinterpret_cast<f32x4 *>(&s_y[group][(threadIdx.x & 31) * 4]) = y;
+        __syncthreads();
+        if (threadIdx.x < 32 && d < p.rank)
+        {
+#pragma unroll
+            for (int k = 1; k < 8; ++k)
+                y = y + *reinterpret_cast<const f32x4 *>(&s_y[k][threadIdx.x * 4]);
             *reinterpret_cast<t4 *>(static_cast<T *>(p.o) + ((size_t)p.row0[e] * p.heads + row) * p.rank + d) =
                 __builtin_convertvector(y * (1.0f / L), t4);
         }
@@ -329,7 +426,7 @@ namespace llamql
         {
             static LdsGrant grant;
             constexpr int WP = 4 / WR;
-            size_t lds = (size_t)32 * WP * (p.rank + 16 / sizeof(T)) * sizeof(T);
+            size_t lds = (size_t)32 * WP * (p.rank + LAT_PAD / sizeof(T)) * sizeof(T) * (QREG && WP == 1 ? 2 : 1);
             const size_t merge = WP > 1 ? (size_t)64 * (NOUT * 16 + 4) * 4 : 0;
             lds = lds > merge ? lds : merge;
             constexpr size_t most = 150 * 1024;
@@ -364,14 +461,14 @@ namespace llamql
             while (pl.wr < 4)
             {
                 const int wp = 4 / pl.wr;
-                if ((size_t)32 * wp * (rank + 16 / elem) * elem <= 140 * 1024)
+                if ((size_t)32 * wp * (rank + LAT_PAD / elem) * elem <= 140 * 1024)
                     break;
                 pl.wr *= 2;
             }
             const int pt = 32 * (4 / pl.wr);
             pl.row_blocks = ceil_div(R, 16 * pl.wr);
             int nsplit = ceil_div(LAT_TARGET, pl.row_blocks * n);
-            const int most = ceil_div(max_len, pt);
+            const int most = ceil_div(max_len, pt > LAT_MIN_STRETCH ? pt : LAT_MIN_STRETCH);
             nsplit = nsplit < most ? nsplit : most;
             pl.chunk = round_up(ceil_div(max_len, nsplit), pt);
             pl.nsplit = ceil_div(max_len, pl.chunk);
@@ -471,8 +568,8 @@ extern "C" bool llam_seq_latent_attention(const void *d_q, const void *d_cache, 
     if (!ok || pl.nsplit == 1)
         return ok;
     if (dtype == LLAM_SEQ_F32)
-        hipLaunchKernelGGL(latent_merge_kernel<float>, dim3(p.rcap, n), dim3(LAT_MERGE_THREADS), 0, st, p);
+        hipLaunchKernelGGL(latent_merge_kernel<float>, dim3(p.rcap, n, ceil_div(rank, LAT_MERGE_COLS)), dim3(256), 0, st, p);
     else
-        hipLaunchKernelGGL(latent_merge_kernel<bf16>, dim3(p.rcap, n), dim3(LAT_MERGE_THREADS), 0, st, p);
+        hipLaunchKernelGGL(latent_merge_kernel<bf16>, dim3(p.rcap, n, ceil_div(rank, LAT_MERGE_COLS)), dim3(256), 0, st, p);
     return launched(fn);
 }

@@ -37,7 +37,10 @@ namespace llamql
         float *mt;      // [rows][heads]: m_t
         float *m0;      // [heads]: m before the portion
         float *prod;    // [chunks][heads][LC][LC]
-        float *num;     // [rows][heads][vdim + 16]
+        float *num;     // [rows][heads][vdim + 16]; decoding: [entries][heads][splits][vdim + 16]
+        int splits;     // decoding: workgroups along dim
+        void *qk;       // T [2][heads][rows of the portion][dim]: scaled q, then k
+        int qk_rows;
     };
 
     __device__ __forceinline__ void memory_gates(const MemoryArgs &p, const float *row, int h, float &i, float &f)
@@ -50,32 +53,25 @@ namespace llamql
     }
 
     // ---- decoding -------------------------------------------------------------------------------
-    // Workgroup = 64 columns of one head's memory of one sequence.
+    // Workgroup = 64 columns of one head's memory of one sequence, and a stretch of its rows.
+    constexpr int STEP_ROWS = 64; // rows of a stretch when there are several
     template <typename T>
     __global__ void __launch_bounds__(256)
         memory_step_kernel(MemoryArgs p)
     {
-        __shared__ float s_q[1024], s_k[1024];
+        __shared__ float s_q[512], s_k[512];
         __shared__ __attribute__((aligned(16))) float s_o[16][64];
-        const int h = blockIdx.y, e = p.entry + blockIdx.z;
+        const int h = blockIdx.y, ei = blockIdx.z, e = p.entry + ei;
+        const int ldv = p.vdim + 16, blocks = (ldv + 63) >> 6;
+        const int split = blockIdx.x / blocks, block = blockIdx.x - split * blocks;
+        const int rows = p.splits > 1 ? STEP_ROWS : p.dim, first = split * rows;
         const int r = p.row0[e], slot = p.slot[e];
         const float *row = p.proj + (size_t)r * p.ldp;
-        const int ldv = p.vdim + 16;
-        const int col = blockIdx.x * 64 + (threadIdx.x & 15) * 4, d0 = threadIdx.x >> 4;
+        const int col = block * 64 + (threadIdx.x & 15) * 4, d0 = threadIdx.x >> 4;
         const bool fresh = p.pos[e] == 0;
-        float *S = p.state + ((size_t)slot * p.heads + h) * p.dim * ldv + col;
+        float *S = p.state + (((size_t)slot * p.heads + h) * p.dim + first) * ldv + col;
         const bool live = col < ldv;
 
-        float gi, gf;
-        memory_gates(p, row, h, gi, gf);
-        const float m_old = fresh ? 0.0f : p.m[slot * p.heads + h];
-        const float m_new = fmaxf(gf + m_old, gi);
-        const float keep = expf(gf + m_old - m_new), take = expf(gi - m_new);
-        for (int d = threadIdx.x; d < p.dim; d += 256)
-        {
-            s_q[d] = rounded<T>(row[h * p.dim + d] * p.q_scale);
-            s_k[d] = rounded<T>(row[(p.heads + h) * p.dim + d]);
-        }
         f32x4 v = {0.0f, 0.0f, 0.0f, 0.0f};
         if (col < p.vdim)
         {
@@ -86,48 +82,73 @@ namespace llamql
         }
         else if (col == p.vdim)
             v[0] = 1.0f;
+        for (int d = threadIdx.x; d < rows; d += 256)
+        {
+            s_q[d] = rounded<T>(row[h * p.dim + first + d] * p.q_scale);
+            s_k[d] = rounded<T>(row[(p.heads + h) * p.dim + first + d]);
+        }
+        constexpr int U = STEP_ROWS / 16; // the first rows are requested before the gates are worked out
+        f32x4 s[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+        {
+            s[u] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+            if (live && !fresh)
+                s[u] = *reinterpret_cast<const f32x4 *>(S + (size_t)(d0 + 16 * u) * ldv);
+        }
+        float gi, gf;
+        memory_gates(p, row, h, gi, gf);
+        const float m_old = fresh ? 0.0f : p.m[slot * p.heads + h];
+        const float m_new = fmaxf(gf + m_old, gi);
+        const float keep = expf(gf + m_old - m_new), take = expf(gi - m_new);
         v = v * take;
         __syncthreads();
         f32x4 o = {0.0f, 0.0f, 0.0f, 0.0f};
         if (live)
-        {
-#pragma unroll 8
-            for (int d = d0; d < p.dim; d += 16)
+            for (int d = d0; d < rows; d += STEP_ROWS)
             {
-                f32x4 *at = reinterpret_cast<f32x4 *>(S + (size_t)d * ldv);
-                f32x4 s = {0.0f, 0.0f, 0.0f, 0.0f};
-                if (!fresh)
-                    s = *at;
-                s = s * keep + v * s_k[d];
-                *at = s;
-                o = o + s * s_q[d];
+                if (d != d0)
+                {
+#pragma unroll
+                    for (int u = 0; u < U; ++u)
+                        s[u] = fresh ? f32x4{0.0f, 0.0f, 0.0f, 0.0f} : *reinterpret_cast<const f32x4 *>(S + (size_t)(d + 16 * u) * ldv);
+                }
+#pragma unroll
+                for (int u = 0; u < U; ++u)
+                {
+                    s[u] = s[u] * keep + v * s_k[d + 16 * u];
+                    *reinterpret_cast<f32x4 *>(S + (size_t)(d + 16 * u) * ldv) = s[u];
+                    o = o + s[u] * s_q[d + 16 * u];
+                }
             }
-        }
         *reinterpret_cast<f32x4 *>(&s_o[d0][(threadIdx.x & 15) * 4]) = o;
         __syncthreads();
-        if (threadIdx.x < 64 && blockIdx.x * 64 + threadIdx.x < ldv)
+        if (threadIdx.x < 64 && block * 64 + threadIdx.x < ldv)
         {
             float sum = 0.0f;
 #pragma unroll
             for (int k = 0; k < 16; ++k)
                 sum += s_o[k][threadIdx.x];
-            p.num[((size_t)r * p.heads + h) * ldv + blockIdx.x * 64 + threadIdx.x] = sum;
+            p.num[(((size_t)ei * p.heads + h) * p.splits + split) * ldv + block * 64 + threadIdx.x] = sum;
         }
     }
 
     // ---- prompts: gates -------------------------------------------------------------------------
+    // A wavefront scans a chunk by itself; the running maximum passes from chunk to chunk by the chunks' totals.
+    constexpr int GATE_WAVES = 16;
     template <int LC>
-    __global__ void __launch_bounds__(64)
+    __global__ void __launch_bounds__(GATE_WAVES * 64)
         memory_gates_kernel(MemoryArgs p)
     {
-        const int h = blockIdx.x, lane = threadIdx.x, e = p.entry;
+        __shared__ double s_total[GATE_WAVES], s_top[GATE_WAVES];
+        const int h = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, e = p.entry;
         const int r0 = p.row0[e], n = p.ntok[e], slot = p.slot[e];
-        double m = p.pos[e] == 0 ? 0.0 : (double)p.m[slot * p.heads + h];
-        if (lane == 0)
-            p.m0[h] = (float)m;
-        for (int t0 = 0; t0 < n; t0 += LC)
+        float m = p.pos[e] == 0 ? 0.0f : p.m[slot * p.heads + h];
+        if (threadIdx.x == 0)
+            p.m0[h] = m;
+        for (int t0 = 0; t0 < n; t0 += GATE_WAVES * LC)
         {
-            const int t = t0 + lane;
+            const int t = t0 + wave * LC + lane;
             const bool in = lane < LC && t < n;
             float gi = -INFINITY, gf = 0.0f;
             if (in)
@@ -149,24 +170,38 @@ namespace llamql
                 if (lane >= off)
                     top = fmax(top, o);
             }
+            __syncthreads();
+            if (lane == 63)
+            {
+                s_total[wave] = F;
+                s_top[wave] = top;
+            }
+            __syncthreads();
             // the running maximum is a 32-bit number of the recurrence
-            const float mt = (float)(F + fmax(m, top));
+            float mine = m;
+            for (int w = 0; w < GATE_WAVES; ++w)
+            {
+                if (w == wave)
+                    mine = m;
+                if (t0 + w * LC < n)
+                    m = (float)(s_total[w] + fmax((double)m, s_top[w]));
+            }
             if (in)
             {
+                const float mt = (float)(F + fmax((double)mine, top));
                 const size_t at = (size_t)(r0 + t) * p.heads + h;
                 p.ga[at] = F - (double)mt;
                 p.a[at] = a;
                 p.mt[at] = mt;
             }
-            const int last = n - t0 < LC ? n - t0 - 1 : LC - 1;
-            m = (double)__shfl(mt, last, 64);
         }
-        if (lane == 0)
-            p.m[slot * p.heads + h] = (float)m;
+        if (threadIdx.x == 0)
+            p.m[slot * p.heads + h] = m;
     }
 
     // ---- prompts: products within a chunk ----------------------------------------------------------
-    // prod[t][j] = e^(F_t + a_j - m_t) (q_t . k_j) for j <= t, else 0.  Wavefront w: rows 16 w ...
+    // prod[t][j] = e^(F_t + a_j - m_t) (q_t . k_j) for j <= t, else 0.  Wavefront w: rows 16 w ...  It also leaves
+    // its rows of q (scaled) and k as T for the walk over the chunks.
     template <typename T, int LC>
     __global__ void __launch_bounds__(LC * 4)
         memory_product_kernel(MemoryArgs p)
@@ -181,6 +216,8 @@ namespace llamql
         const int r0 = p.row0[e] + chunk * LC;
         auto row = [&](int t) { return p.proj + (size_t)(r0 + (t < n ? t : n - 1)) * p.ldp; };
         const float *q = row(wave * 16 + c) + h * p.dim + 8 * g;
+        T *qk = static_cast<T *>(p.qk) + ((size_t)h * p.qk_rows + chunk * LC + wave * 16 + c) * p.dim + 8 * g;
+        const size_t k_after = (size_t)p.heads * p.qk_rows * p.dim;
         const float *k[LC / 16];
 #pragma unroll
         for (int j = 0; j < LC / 16; ++j)
@@ -193,12 +230,15 @@ namespace llamql
         {
             V a[1], b[1];
             split_pieces<T, 1>(Operand<float>::load(q + s) * p.q_scale, a);
+            *reinterpret_cast<V *>(qk + s) = a[0];
 #pragma unroll
             for (int j = 0; j < LC / 16; ++j)
                 if (j <= wave)
                 {
                     split_pieces<T, 1>(Operand<float>::load(k[j] + s), b);
                     acc[j] = O::mma(a[0], b[0], acc[j]);
+                    if (j == wave)
+                        *reinterpret_cast<V *>(qk + k_after + s) = b[0];
                 }
         }
         float *out = p.prod + ((size_t)chunk * p.heads + h) * LC * LC;
@@ -221,6 +261,8 @@ namespace llamql
 
     // ---- prompts: the walk over the chunks ----------------------------------------------------------
     // Workgroup = up to four wavefronts of 16 columns each, of one head.  DT: 16-row tiles of S (dim <= 16 DT).
+    // What the next chunk needs from memory (q and k for the LDS, this column's values, the products) is
+    // requested before the matrix work of the current one.
     template <typename T, int LC, int DT>
     __global__ void __launch_bounds__(256)
         memory_chunk_kernel(MemoryArgs p)
@@ -230,6 +272,9 @@ namespace llamql
         typedef T t4 __attribute__((ext_vector_type(4)));
         constexpr int NP = O::PIECES;
         constexpr int LPAD = 16 / sizeof(T);
+        constexpr int TPR = 256 / LC;                            // threads of a row when q and k are staged
+        constexpr int LOADS = DT * 16 * (int)sizeof(T) / 16 / TPR; // 16-byte pieces of a row per thread
+        constexpr bool AHEAD = LOADS <= 8;                       // staged rows of the next chunk fit the registers
         extern __shared__ __attribute__((aligned(16))) char smem[];
         __shared__ float s_carry[LC], s_gate[LC]; // e^(F_t + m0 - m_t), e^(F_end + a_j - m_end)
         const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
@@ -257,35 +302,101 @@ namespace llamql
             }
         }
 
+        const int srow = threadIdx.x / TPR, sseg = threadIdx.x % TPR, pieces = p.dim * (int)sizeof(T) / 16;
+        const T *qrows = static_cast<const T *>(p.qk) + (size_t)h * p.qk_rows * p.dim;
+        const T *krows = qrows + (size_t)p.heads * p.qk_rows * p.dim;
+        u32x4 hq[AHEAD ? LOADS : 1], hk[AHEAD ? LOADS : 1];
+        f32x8 hv[LC / 32];
+        double h_ga = 0.0, h_a = 0.0, h_end = 0.0;
+        float h_mt = 0.0f;
+        auto request = [&](int t0) __attribute__((always_inline)) {
+            const int n = ntok - t0 < LC ? ntok - t0 : LC;
+            const int r0 = row0 + t0;
+            if constexpr (AHEAD)
+            {
+                // (the product kernel wrote whole chunks: rows past the portion repeat its last one)
+                const u32x4 *q = reinterpret_cast<const u32x4 *>(qrows + (size_t)(t0 + srow) * p.dim) + sseg;
+                const u32x4 *k = reinterpret_cast<const u32x4 *>(krows + (size_t)(t0 + srow) * p.dim) + sseg;
+#pragma unroll
+                for (int i = 0; i < LOADS; ++i)
+                {
+                    const int at = sseg + i * TPR < pieces ? i * TPR : 0;
+                    hq[i] = q[at];
+                    hk[i] = k[at];
+                }
+            }
+            const size_t end = (size_t)(r0 + n - 1) * p.heads + h;
+            const int t = threadIdx.x & (LC - 1);
+            const size_t at = (size_t)(r0 + (t < n ? t : n - 1)) * p.heads + h;
+            h_ga = p.ga[at];
+            h_a = p.a[at];
+            h_end = p.ga[end];
+            h_mt = p.mt[end];
+#pragma unroll
+            for (int s = 0; s < LC / 32; ++s)
+#pragma unroll
+                for (int j = 0; j < 8; ++j)
+                {
+                    const int tt = 32 * s + 8 * g + j;
+                    hv[s][j] = ones || !live ? 0.0f
+                                             : p.proj[(size_t)(r0 + (tt < n ? tt : n - 1)) * p.ldp + (size_t)p.heads * 2 * p.dim + h * p.vdim + col];
+                }
+        };
+        request(0);
         float m0 = p.m0[h];
         for (int t0 = 0; t0 < ntok; t0 += LC)
         {
             const int n = ntok - t0 < LC ? ntok - t0 : LC;
             const int r0 = row0 + t0;
-            const size_t end = (size_t)(r0 + n - 1) * p.heads + h;
-            const double g_end = p.ga[end];
-            const float decay = expf((float)(g_end + (double)m0));
+            const float decay = expf((float)(h_end + (double)m0));
+            const float m_end = h_mt;
             __syncthreads();
             if (threadIdx.x < LC)
             {
                 const int t = threadIdx.x;
-                const size_t at = (size_t)(r0 + (t < n ? t : n - 1)) * p.heads + h;
-                s_carry[t] = t < n ? expf((float)(p.ga[at] + (double)m0)) : 0.0f;
-                s_gate[t] = t < n ? expf((float)(g_end + p.a[at])) : 0.0f;
+                s_carry[t] = t < n ? expf((float)(h_ga + (double)m0)) : 0.0f;
+                s_gate[t] = t < n ? expf((float)(h_end + h_a)) : 0.0f;
             }
-            // q (scaled) and k of the chunk, as T: 16 threads a row
-            for (int t = threadIdx.x >> 4; t < LC; t += 16)
             {
-                const float *row = p.proj + (size_t)(r0 + (t < n ? t : n - 1)) * p.ldp + h * p.dim;
-                for (int d = (threadIdx.x & 15) * 4; d < p.dim; d += 64)
+                u32x4 *dq = reinterpret_cast<u32x4 *>(sq + srow * ld) + sseg, *dk = reinterpret_cast<u32x4 *>(sk + srow * ld) + sseg;
+                if constexpr (AHEAD)
                 {
-                    const f32x4 q = *reinterpret_cast<const f32x4 *>(row + d) * p.q_scale;
-                    const f32x4 k = *reinterpret_cast<const f32x4 *>(row + (size_t)p.heads * p.dim + d);
-                    *reinterpret_cast<t4 *>(sq + t * ld + d) = __builtin_convertvector(q, t4);
-                    *reinterpret_cast<t4 *>(sk + t * ld + d) = __builtin_convertvector(k, t4);
+#pragma unroll
+                    for (int i = 0; i < LOADS; ++i)
+                        if (sseg + i * TPR < pieces)
+                        {
+                            dq[i * TPR] = hq[i];
+                            dk[i * TPR] = hk[i];
+                        }
+                }
+                else
+                {
+                    const u32x4 *q = reinterpret_cast<const u32x4 *>(qrows + (size_t)(t0 + srow) * p.dim) + sseg;
+                    const u32x4 *k = reinterpret_cast<const u32x4 *>(krows + (size_t)(t0 + srow) * p.dim) + sseg;
+#pragma unroll 4
+                    for (int i = 0; sseg + i < pieces; i += TPR)
+                    {
+                        dq[i] = q[i];
+                        dk[i] = k[i];
+                    }
                 }
             }
+            f32x8 x[LC / 32];
+#pragma unroll
+            for (int s = 0; s < LC / 32; ++s)
+                x[s] = hv[s];
             __syncthreads();
+            // the chunk's products, 16 rows at a time (a row block needs columns up to its own)
+            const float *prod = p.prod + ((size_t)(t0 / LC) * p.heads + h) * LC * LC;
+            f32x8 w[LC / 16][LC / 32];
+#pragma unroll
+            for (int i = 0; i < LC / 16; ++i)
+#pragma unroll
+                for (int s = 0; s < LC / 32; ++s)
+                    if (32 * s <= 16 * i + 15)
+                        w[i][s] = Operand<float>::load(prod + (16 * i + c) * LC + 32 * s + 8 * g);
+            if (t0 + LC < ntok)
+                request(t0 + LC);
             if (live)
             {
                 // values of this column, as they are and gated
@@ -293,24 +404,20 @@ namespace llamql
 #pragma unroll
                 for (int s = 0; s < LC / 32; ++s)
                 {
-                    f32x8 x;
-#pragma unroll
-                    for (int j = 0; j < 8; ++j)
+                    if (ones)
                     {
-                        const int t = 32 * s + 8 * g + j;
-                        if (ones)
-                            x[j] = c == 0 && t < n ? 1.0f : 0.0f;
-                        else
-                            x[j] = p.proj[(size_t)(r0 + (t < n ? t : n - 1)) * p.ldp + (size_t)p.heads * 2 * p.dim + h * p.vdim + col];
+#pragma unroll
+                        for (int j = 0; j < 8; ++j)
+                            x[s][j] = c == 0 && 32 * s + 8 * g + j < n ? 1.0f : 0.0f;
                     }
                     V one[1];
-                    split_pieces<T, 1>(x, one);
+                    split_pieces<T, 1>(x[s], one);
                     v[s] = one[0];
-                    x = __builtin_convertvector(one[0], f32x8);
+                    f32x8 y;
 #pragma unroll
                     for (int j = 0; j < 8; ++j)
-                        x[j] *= s_gate[32 * s + 8 * g + j];
-                    split_pieces<T, NP>(x, gv[s]);
+                        y[j] = (float)one[0][j] * s_gate[32 * s + 8 * g + j];
+                    split_pieces<T, NP>(y, gv[s]);
                 }
                 // carried part: q . S
                 f32x4 out[LC / 16];
@@ -321,37 +428,43 @@ namespace llamql
                 for (int t = 0; t < DT; t += 2)
                     if (t < dtiles)
                     {
-                        V b[NP];
+                        V b[NP], a[LC / 16];
                         split_pieces<T, NP>(__builtin_shufflevector(S[t], S[t + 1], 0, 1, 2, 3, 4, 5, 6, 7), b);
 #pragma unroll
                         for (int i = 0; i < LC / 16; ++i)
                         {
                             const T *qr = sq + (16 * i + c) * ld + 16 * t + 4 * g;
                             const t4 lo = *reinterpret_cast<const t4 *>(qr), hi = *reinterpret_cast<const t4 *>(qr + 16);
-                            const V a = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-#pragma unroll
-                            for (int k = 0; k < NP; ++k)
-                                out[i] = O::mma(a, b[k], out[i]);
+                            a[i] = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
                         }
+#pragma unroll
+                        for (int k = 0; k < NP; ++k)
+#pragma unroll
+                            for (int i = 0; i < LC / 16; ++i)
+                                out[i] = O::mma(a[i], b[k], out[i]);
                     }
                 // plus the chunk's own tokens
-                const float *prod = p.prod + ((size_t)(t0 / LC) * p.heads + h) * LC * LC;
 #pragma unroll
                 for (int i = 0; i < LC / 16; ++i)
                 {
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
                         out[i][r] *= s_carry[16 * i + 4 * g + r];
+                }
 #pragma unroll
-                    for (int s = 0; s < LC / 32; ++s)
+                for (int s = 0; s < LC / 32; ++s)
+#pragma unroll
+                    for (int i = 0; i < LC / 16; ++i)
                         if (32 * s <= 16 * i + 15)
                         {
-                            V w[NP];
-                            split_pieces<T, NP>(Operand<float>::load(prod + (16 * i + c) * LC + 32 * s + 8 * g), w);
+                            V q[NP];
+                            split_pieces<T, NP>(w[i][s], q);
 #pragma unroll
                             for (int k = 0; k < NP; ++k)
-                                out[i] = O::mma(w[k], v[s], out[i]);
+                                out[i] = O::mma(q[k], v[s], out[i]);
                         }
+#pragma unroll
+                for (int i = 0; i < LC / 16; ++i)
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
                     {
@@ -359,7 +472,6 @@ namespace llamql
                         if (t < n)
                             p.num[((size_t)(r0 + t) * p.heads + h) * ldv + col] = out[i][r];
                     }
-                }
                 // S of the next chunk
 #pragma unroll
                 for (int t = 0; t < DT; ++t)
@@ -368,17 +480,27 @@ namespace llamql
 #pragma unroll
                         for (int r = 0; r < 4; ++r)
                             S[t][r] *= decay;
+                    }
+#pragma unroll
+                for (int t = 0; t < DT; t += 4)
+                    if (t < dtiles)
+                    {
 #pragma unroll
                         for (int s = 0; s < LC / 32; ++s)
                         {
-                            const V k = load_columns(sk + 32 * s * ld + 16 * t, ld, lane);
+                            V k[4];
+#pragma unroll
+                            for (int u = 0; u < 4; ++u)
+                                k[u] = load_columns(sk + 32 * s * ld + 16 * (t + u), ld, lane);
 #pragma unroll
                             for (int i = 0; i < NP; ++i)
-                                S[t] = O::mma(k, gv[s][i], S[t]);
+#pragma unroll
+                                for (int u = 0; u < 4; ++u)
+                                    S[t + u] = O::mma(k[u], gv[s][i], S[t + u]);
                         }
                     }
             }
-            m0 = p.mt[end];
+            m0 = m_end;
         }
         if (live)
         {
@@ -405,7 +527,8 @@ namespace llamql
         const int r = DECODE ? p.row0[e] : p.row0[e] + blockIdx.y;
         const float *row = p.proj + (size_t)r * p.ldp;
         const int ldv = p.vdim + 16;
-        const float *num = p.num + ((size_t)r * p.heads + h) * ldv;
+        const int splits = DECODE ? p.splits : 1;
+        const float *num = p.num + ((size_t)(DECODE ? blockIdx.y : r) * p.heads + h) * splits * ldv;
         float m;
         if (DECODE)
         {
@@ -419,30 +542,50 @@ namespace llamql
         }
         else
             m = p.mt[(size_t)r * p.heads + h];
-        const float inv = 1.0f / (fmaxf(fabsf(num[p.vdim]), expf(-m)) + 1e-6f);
+        // columns 4 threadIdx.x .. + 3, and 512 further on (the first are kept for the second pass)
+        auto total = [&](int d) {
+            f32x4 o = *reinterpret_cast<const f32x4 *>(num + d);
+            for (int k = 1; k < splits; ++k)
+                o = o + *reinterpret_cast<const f32x4 *>(num + (size_t)k * ldv + d);
+            return o;
+        };
+        const float inv = 1.0f / (fmaxf(fabsf(total(p.vdim)[0]), expf(-m)) + 1e-6f);
+        const int d0 = threadIdx.x * 4;
+        f32x4 kept = {0.0f, 0.0f, 0.0f, 0.0f};
         float sum = 0.0f;
-        for (int d = threadIdx.x; d < p.vdim; d += 128)
+        for (int d = d0; d < p.vdim; d += 512)
         {
-            const float o = num[d] * inv;
-            sum += o * o;
+            const f32x4 o = total(d) * inv;
+            if (d == d0)
+                kept = o;
+            sum += o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
         }
         sum = block_sum<128>(sum, s_sum);
-        const float scale = inv / sqrtf(sum / (float)p.vdim_real + p.eps);
+        const float scale = 1.0f / sqrtf(sum / (float)p.vdim_real + p.eps);
         const float *gate = row + (size_t)p.heads * (2 * p.dim + p.vdim) + h * p.vdim;
+        typedef T t4 __attribute__((ext_vector_type(4)));
         T *y = static_cast<T *>(p.y) + ((size_t)r * p.heads + h) * p.vdim;
-        for (int d = threadIdx.x; d < p.vdim; d += 128)
-            y[d] = (T)(num[d] * scale * p.norm[h * p.vdim + d] * sigmoidf(gate[d]));
+        for (int d = d0; d < p.vdim; d += 512)
+        {
+            f32x4 o = (d == d0 ? kept : total(d) * inv) * scale * *reinterpret_cast<const f32x4 *>(p.norm + h * p.vdim + d);
+            const f32x4 z = *reinterpret_cast<const f32x4 *>(gate + d);
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+                o[k] *= sigmoidf(z[k]);
+            *reinterpret_cast<t4 *>(y + d) = __builtin_convertvector(o, t4);
+        }
     }
 
     namespace
     {
         constexpr int LC16 = 64, LC32 = 32; // chunk lengths of the two number formats
+        constexpr int STEP_SPLIT_ENTRIES = 32; // sequences up to which a decoding step splits the rows of S (in at most 8)
 
         struct MemoryScratch
         {
-            size_t ga, a, mt, m0, prod, num, total;
+            size_t ga, a, mt, m0, prod, num, qk, total;
         };
-        MemoryScratch memory_scratch(int rows, int heads, int vdim)
+        MemoryScratch memory_scratch(int rows, int heads, int dim, int vdim)
         {
             MemoryScratch s{};
             size_t at = 0;
@@ -456,7 +599,9 @@ namespace llamql
             s.mt = take((size_t)rows * heads * 4);
             s.m0 = take((size_t)heads * 4);
             s.prod = take((size_t)round_up(rows, LC16) * heads * LC16 * 4);
-            s.num = take((size_t)rows * heads * (vdim + 16) * 4);
+            const size_t outs = (size_t)(rows > STEP_SPLIT_ENTRIES * 8 ? rows : STEP_SPLIT_ENTRIES * 8);
+            s.num = take(outs * heads * (vdim + 16) * 4);
+            s.qk = take((size_t)2 * heads * round_up(rows, LC16) * dim * 4);
             s.total = at;
             return s;
         }
@@ -487,15 +632,15 @@ namespace llamql
         {
             // rows of the step are absolute, so the offsets are those of the whole buffer: the largest
             // row count whose scratch fits
-            const size_t per = memory_scratch(64, p.heads, p.vdim).total;
-            int rows = (int)(scratch_bytes / per) * 64;
-            while (memory_scratch(rows + 64, p.heads, p.vdim).total <= scratch_bytes)
+            int rows = 64;
+            while (memory_scratch(rows + 64, p.heads, p.dim, p.vdim).total <= scratch_bytes)
                 rows += 64;
-            const MemoryScratch at = memory_scratch(rows, p.heads, p.vdim);
+            const MemoryScratch at = memory_scratch(rows, p.heads, p.dim, p.vdim);
             char *s = static_cast<char *>(d_scratch);
             p.ga = reinterpret_cast<double *>(s + at.ga), p.a = reinterpret_cast<double *>(s + at.a);
             p.mt = reinterpret_cast<float *>(s + at.mt), p.m0 = reinterpret_cast<float *>(s + at.m0);
             p.prod = reinterpret_cast<float *>(s + at.prod), p.num = reinterpret_cast<float *>(s + at.num);
+            p.qk = s + at.qk, p.qk_rows = rows;
         }
 
         template <typename T, int LC, int DT>
@@ -511,7 +656,7 @@ namespace llamql
         template <typename T, int LC>
         bool prefill_run(const char *fn, const MemoryArgs &p, int ntok, hipStream_t st)
         {
-            hipLaunchKernelGGL(memory_gates_kernel<LC>, dim3(p.heads), dim3(64), 0, st, p);
+            hipLaunchKernelGGL(memory_gates_kernel<LC>, dim3(p.heads), dim3(GATE_WAVES * 64), 0, st, p);
             if (!launched(fn))
                 return false;
             hipLaunchKernelGGL((memory_product_kernel<T, LC>), dim3(ceil_div(ntok, LC), p.heads), dim3(LC * 4), 0, st, p);
@@ -525,9 +670,10 @@ namespace llamql
             return launched(fn);
         }
         template <typename T>
-        bool decode_run(const char *fn, const MemoryArgs &p, int n, hipStream_t st)
+        bool decode_run(const char *fn, MemoryArgs p, int n, hipStream_t st)
         {
-            hipLaunchKernelGGL(memory_step_kernel<T>, dim3(ceil_div(p.vdim + 16, 64), p.heads, n), dim3(256), 0, st, p);
+            p.splits = n <= STEP_SPLIT_ENTRIES ? p.dim / STEP_ROWS : 1;
+            hipLaunchKernelGGL(memory_step_kernel<T>, dim3(ceil_div(p.vdim + 16, 64) * p.splits, p.heads, n), dim3(256), 0, st, p);
             if (!launched(fn))
                 return false;
             hipLaunchKernelGGL((memory_output_kernel<T, true>), dim3(p.heads, n), dim3(128), 0, st, p);
@@ -538,11 +684,11 @@ namespace llamql
 
 using namespace llamql;
 
-extern "C" size_t llam_seq_memory_scratch_bytes(int max_rows, int heads, int vdim)
+extern "C" size_t llam_seq_memory_scratch_bytes(int max_rows, int heads, int dim, int vdim)
 {
-    if (max_rows < 1 || heads < 1 || vdim < 1)
+    if (max_rows < 1 || heads < 1 || dim < 1 || vdim < 1)
         return 0;
-    return memory_scratch(round_up(max_rows, LC16), heads, vdim).total;
+    return memory_scratch(round_up(max_rows, LC16), heads, dim, vdim).total;
 }
 
 extern "C" bool llam_seq_memory_decode(const llam_seq_memory_args *a, const llam_seq_entries *e, int first, int n,
@@ -556,7 +702,7 @@ extern "C" bool llam_seq_memory_decode(const llam_seq_memory_args *a, const llam
         return true;
     if (!memory_args(fn, a, e, d_scratch, dtype, p))
         return false;
-    if (llam_seq_memory_scratch_bytes(first + n, p.heads, p.vdim) > scratch_bytes)
+    if (llam_seq_memory_scratch_bytes(first + n, p.heads, p.dim, p.vdim) > scratch_bytes)
         return fail(fn, "scratch too small");
     p.entry = first;
     place_scratch(p, d_scratch, scratch_bytes);
@@ -576,7 +722,7 @@ extern "C" bool llam_seq_memory_prefill(const llam_seq_memory_args *a, const lla
         return true;
     if (!memory_args(fn, a, e, d_scratch, dtype, p))
         return false;
-    if (llam_seq_memory_scratch_bytes(ntok, p.heads, p.vdim) > scratch_bytes)
+    if (llam_seq_memory_scratch_bytes(ntok, p.heads, p.dim, p.vdim) > scratch_bytes)
         return fail(fn, "scratch too small");
     p.entry = entry;
     place_scratch(p, d_scratch, scratch_bytes);

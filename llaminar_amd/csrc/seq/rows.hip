@@ -10,9 +10,9 @@ namespace llamql
         seq_embed_kernel(const bf16 *__restrict__ table, int vocab, int width, const int32_t *__restrict__ ids,
                          float *__restrict__ x, int ldx)
     {
-        const int m = blockIdx.x, id = ids[m];
+        const int m = blockIdx.y, id = ids[m], c = blockIdx.x * ROW_THREADS + threadIdx.x;
         const bool ok = id >= 0 && id < vocab;
-        for (int c = threadIdx.x; c < ldx; c += ROW_THREADS)
+        if (c < ldx)
             x[(size_t)m * ldx + c] = ok && c < width ? (float)table[(size_t)id * width + c] : 0.0f;
     }
 
@@ -70,7 +70,7 @@ namespace llamql
     // Few rows.  Workgroup = 16 outputs of one expert of one token.  All workgroups choose the
     // token's experts for themselves from the logits; the first of a token records the choice for
     // the down projections.
-    constexpr int EXPERT_WAVES = 4;
+    constexpr int EXPERT_WAVES = 8;
     template <typename T>
     __global__ void __launch_bounds__(EXPERT_WAVES * 64)
         expert_up_small_kernel(ExpertArgs p)
@@ -152,47 +152,55 @@ namespace llamql
         expert_down_small_kernel(ExpertArgs p)
     {
         using O = Operand<T>;
+        using V = typename O::V;
         __shared__ __attribute__((aligned(16))) float s_red[EXPERT_WAVES][64][4];
         const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4;
+        __shared__ int s_ids[64];
+        __shared__ float s_weights[65];
         const int tile = blockIdx.x, m = blockIdx.y;
         const int esteps = p.ff >> 5, ssteps = p.shared_ff >> 5;
-        const int routed = p.top * esteps, total = routed + ssteps;
+        const int total = p.top * esteps + ssteps;
+        if (threadIdx.x <= p.top)
+        {
+            if (threadIdx.x < p.top)
+                s_ids[threadIdx.x] = p.ids[m * p.top + threadIdx.x];
+            s_weights[threadIdx.x] = p.weights[m * (p.top + 1) + threadIdx.x];
+        }
         const T *act = static_cast<const T *>(p.act) + (size_t)m * (p.top * p.ff + p.shared_ff) + 8 * g;
-        const int *ids = p.ids + m * p.top;
-        const float *weights = p.weights + m * (p.top + 1);
+        __syncthreads();
         f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
-        constexpr int U = 4;
+        constexpr int U = 8;
+        // the wavefront's place in the list: step s is step `in` of expert `job`
+        int job = 0, in = wave;
         for (int s0 = wave; s0 < total; s0 += EXPERT_WAVES * U)
         {
             u32x4 raw[U];
+            V b[U];
             float scale[U];
 #pragma unroll
             for (int u = 0; u < U; ++u)
             {
-                int s = s0 + u * EXPERT_WAVES;
-                s = s < total ? s : s0;
-                if (s < routed)
+                const int s = s0 + u * EXPERT_WAVES;
+                while (job < p.top && in >= esteps)
                 {
-                    const int job = s / esteps;
-                    raw[u] = weight_tile(p.down + (size_t)ids[job] * p.down_stride, tile, esteps, lane)[(size_t)(s - job * esteps) * 64];
-                    scale[u] = weights[job];
+                    in -= esteps;
+                    ++job;
                 }
-                else
-                {
-                    raw[u] = weight_tile(p.shared_down, tile, ssteps, lane)[(size_t)(s - routed) * 64];
-                    scale[u] = weights[p.top];
-                }
+                const bool live = s < total;
+                const int id = __builtin_amdgcn_readfirstlane(s_ids[job < p.top ? job : 0]);
+                // (past the end: any step of the first expert, with weight zero)
+                const u32x4 *w = job < p.top || !live ? weight_tile(p.down + (size_t)id * p.down_stride, tile, esteps, lane)
+                                             : weight_tile(p.shared_down, tile, ssteps, lane);
+                raw[u] = w[(size_t)(live ? in : 0) * 64];
+                b[u] = O::load(act + (size_t)(live ? s : 0) * 32);
+                scale[u] = live ? s_weights[job < p.top ? job : p.top] : 0.0f;
+                in += EXPERT_WAVES;
             }
 #pragma unroll
             for (int u = 0; u < U; ++u)
             {
-                const int s = s0 + u * EXPERT_WAVES;
-                if (s < total)
-                {
-                    const f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
-                    const f32x4 d = O::mma(O::from_weights(raw[u]), O::load(act + (size_t)s * 32), zero);
-                    acc = acc + d * scale[u];
-                }
+                const f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
+                acc = acc + O::mma(O::from_weights(raw[u]), b[u], zero) * scale[u];
             }
         }
         *reinterpret_cast<f32x4 *>(s_red[wave][lane]) = acc;
@@ -230,14 +238,15 @@ namespace llamql
 
     // ... the (token, choice) pairs are put in order of their expert, each expert's in the order of
     // the tokens: one workgroup per expert counts the pairs of lower experts and places its own
-    __global__ void __launch_bounds__(ROW_THREADS)
+    constexpr int GROUP_THREADS = 1024;
+    __global__ void __launch_bounds__(GROUP_THREADS)
         expert_group_kernel(const int *__restrict__ ids, int pairs, int experts, int *__restrict__ offset,
                             int *__restrict__ order, int *__restrict__ place)
     {
-        __shared__ int s_low[ROW_THREADS / 64], s_own[ROW_THREADS / 64];
+        __shared__ int s_low[GROUP_THREADS / 64], s_own[GROUP_THREADS / 64];
         const int e = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
         int low = 0;
-        for (int i = threadIdx.x; i < pairs; i += ROW_THREADS)
+        for (int i = threadIdx.x; i < pairs; i += GROUP_THREADS)
             low += ids[i] < e;
 #pragma unroll
         for (int off = 32; off > 0; off >>= 1)
@@ -246,7 +255,7 @@ namespace llamql
             s_low[wave] = low;
         __syncthreads();
         int base = 0;
-        for (int w = 0; w < ROW_THREADS / 64; ++w)
+        for (int w = 0; w < GROUP_THREADS / 64; ++w)
             base += s_low[w];
         if (threadIdx.x == 0)
         {
@@ -254,7 +263,7 @@ namespace llamql
             if (e == experts - 1)
                 offset[experts] = pairs;
         }
-        for (int i0 = 0; i0 < pairs; i0 += ROW_THREADS)
+        for (int i0 = 0; i0 < pairs; i0 += GROUP_THREADS)
         {
             const int i = i0 + threadIdx.x;
             const bool own = i < pairs && ids[i] == e;
@@ -263,7 +272,7 @@ namespace llamql
                 s_own[wave] = __popcll(mask);
             __syncthreads();
             int at = base;
-            for (int w = 0; w < ROW_THREADS / 64; ++w)
+            for (int w = 0; w < GROUP_THREADS / 64; ++w)
             {
                 if (w < wave)
                     at += s_own[w];
@@ -351,7 +360,7 @@ namespace llamql
             hipLaunchKernelGGL(expert_route_kernel, dim3(ceil_div(M, ROW_THREADS / 64)), dim3(ROW_THREADS), 0, st, p, M);
             if (!launched(fn))
                 return false;
-            hipLaunchKernelGGL(expert_group_kernel, dim3(p.experts), dim3(ROW_THREADS), 0, st, p.ids, M * p.top, p.experts,
+            hipLaunchKernelGGL(expert_group_kernel, dim3(p.experts), dim3(GROUP_THREADS), 0, st, p.ids, M * p.top, p.experts,
                                offset, order, place);
             if (!launched(fn))
                 return false;
@@ -401,7 +410,9 @@ extern "C" bool llam_seq_embed(const void *d_table, int vocab, int width, const 
         return fail(fn, "null pointer");
     if (!set_device(fn, device_id))
         return false;
-    hipLaunchKernelGGL(seq_embed_kernel, dim3(M), dim3(ROW_THREADS), 0, as_stream(stream),
+    if (M > 65535)
+        return fail(fn, "M=%d rows", M);
+    hipLaunchKernelGGL(seq_embed_kernel, dim3(ceil_div(ldx, ROW_THREADS), M), dim3(ROW_THREADS), 0, as_stream(stream),
                        static_cast<const bf16 *>(d_table), vocab, width, d_ids, d_x, ldx);
     return launched(fn);
 }

@@ -423,7 +423,7 @@ extern "C" bool llam_seqm_set_globals(void *model, const llam_seqm_globals *g)
         else
         {
             n_in = std::max(n_in, (size_t)pad((int)(2 * H * (dp + vp) + 2 * H), 16));
-            scratch = std::max(scratch, llam_seq_memory_scratch_bytes(std::max(c.max_rows, c.slots), w.heads, (int)vp));
+            scratch = std::max(scratch, llam_seq_memory_scratch_bytes(std::max(c.max_rows, c.slots), w.heads, (int)dp, (int)vp));
         }
         if (w.ffn == LLAM_FFN_GATED)
             act = std::max(act, (size_t)P(w.ff));

@@ -84,7 +84,7 @@ SIGNATURES = {
     "llam_seq_latent_scratch_floats": (c_size_t, [c_int, c_int, c_int, c_int, c_int]),
     "llam_seq_latent_attention": (c_bool, [c_void_p, c_void_p, POINTER(Entries), c_int, c_int, c_int, c_int, c_int,
                                            c_int, c_int, c_float, c_void_p, c_void_p, c_size_t, c_int, c_int, c_void_p]),
-    "llam_seq_memory_scratch_bytes": (c_size_t, [c_int, c_int, c_int]),
+    "llam_seq_memory_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int]),
     "llam_seq_memory_decode": (c_bool, [POINTER(MemoryArgs), POINTER(Entries), c_int, c_int, c_void_p, c_size_t, c_int,
                                         c_int, c_void_p]),
     "llam_seq_memory_prefill": (c_bool, [POINTER(MemoryArgs), POINTER(Entries), c_int, c_int, c_void_p, c_size_t, c_int,
