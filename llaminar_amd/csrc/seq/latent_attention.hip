@@ -20,11 +20,37 @@ namespace llamql
 {
     constexpr int LAT_THREADS = 512;
     constexpr int LAT_TARGET = 256; // workgroups aimed at before rows are no longer split
+    // positions of a turn that a group takes: 64 where it has the row block to itself and the registers allow
+    constexpr int lat_group(int nout, bool qreg, int wr) { return wr == 4 && nout < 32 && qreg ? 64 : 32; }
     constexpr int LAT_MIN_STRETCH = 64; // positions: shorter stretches cost more in partial results than they gain
 
-    constexpr int LAT_PAD = 32;         // bytes between staged rows: both kinds of LDS read spread over the banks
+    // Staged rows lie without padding (a row is a multiple of all 32 banks), their 16-byte pieces permuted by the row:
+    // piece q of row r is at q ^ lat_swizzle(r).  Eight rows' equal pieces then lie in different banks (the
+    // scores' reads), and so do two neighbouring pieces of four rows (the transposing reads).
+    __device__ __forceinline__ int lat_swizzle(int r) { return ((r & 3) << 1) | ((r >> 2) & 1); }
 
     __device__ __forceinline__ float fast_exp(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+
+    // Columns 16 (tile0 + t) .. + 15 of 32 staged rows as a second operand (see load_columns); tile0 a multiple of 4
+    __device__ __forceinline__ bf16x8 lat_columns(const bf16 *rows, int ld, int tile0, int t, int lane)
+    {
+        typedef __attribute__((address_space(3))) bf16x4 *lds4;
+        const int i = lane & 15, r = 8 * (lane >> 4) + (i >> 2);
+        const int piece = (2 * t + ((i & 3) >> 1)) & 7;
+        const bf16 *p = rows + r * ld + 16 * tile0 + ((2 * t) >> 3) * 64 + (i & 1) * 4;
+        const bf16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds4)(p + (piece ^ ((i >> 2) << 1)) * 8));
+        const bf16x4 b = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds4)(p + 4 * ld + (piece ^ (((i >> 2) << 1) | 1)) * 8));
+        return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+    }
+    __device__ __forceinline__ f32x8 lat_columns(const float *rows, int ld, int tile0, int t, int lane)
+    {
+        const int c = lane & 15, piece = 4 * (tile0 + t) + (c >> 2);
+        f32x8 v;
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            v[j] = rows[(8 * (lane >> 4) + j) * ld + (piece ^ lat_swizzle(j)) * 4 + (c & 3)];
+        return v;
+    }
 
     struct LatentArgs
     {
@@ -39,18 +65,19 @@ namespace llamql
 
     // NOUT: 16-column output tiles of a row block, half of them per wavefront.  QREG: the query rows stay in
     // registers (rank <= 16 NOUT); otherwise they are read again for every turn and blockIdx.z also counts
-    // slices of the output.
-    template <typename T, int NOUT, bool QREG, int WR>
+    // slices of the output.  FULL: the rank is 16 NOUT exactly, so that no product hangs on a condition.
+    template <typename T, int NOUT, bool QREG, bool FULL, int WR>
     __global__ void __launch_bounds__(LAT_THREADS)
         latent_attention_kernel(LatentArgs p)
     {
         using O = Operand<T>;
         using V = typename O::V;
         typedef T t4 __attribute__((ext_vector_type(4)));
-        constexpr int WP = 4 / WR, PT = 32 * WP;
-        constexpr int LPAD = LAT_PAD / sizeof(T);
+        constexpr int WP = 4 / WR;
+        constexpr int PG = lat_group(NOUT, QREG, WR), PT = PG * WP; // positions of a group, of a turn
+        constexpr int PS = PG / 32;                               // steps of 32 positions
         constexpr int PW = sizeof(T) == 2 ? 2 : 1; // pieces of a softmax weight
-        constexpr int SLD = 36;
+        constexpr int SLD = PG + 4;
         constexpr int NT = NOUT / 2;               // output tiles of a wavefront
         extern __shared__ __attribute__((aligned(16))) char smem[];
         __shared__ __attribute__((aligned(16))) float s_s[4][16 * SLD];
@@ -71,38 +98,39 @@ namespace llamql
             return;
         const int k1 = k0 + p.chunk < kmax + 1 ? k0 + p.chunk : kmax + 1;
 
-        const int ksteps = p.rank >> 5;
-        const int ld = p.rank + LPAD;
-        const T *cache = static_cast<const T *>(p.cache) + (size_t)p.slot[e] * p.cap * p.rank;
+        const int rank = FULL ? 16 * NOUT : p.rank;
+        const int ksteps = rank >> 5;
+        const int ld = rank;
+        const T *cache = static_cast<const T *>(p.cache) + (size_t)p.slot[e] * p.cap * rank;
 
         // The cache rows of a turn: TPR threads a row.  With two buffers the next turn's rows are requested
         // before this turn's products and put down in the middle of them.
         constexpr int TPR = LAT_THREADS / PT;
         constexpr int LOADS = NOUT * (int)sizeof(T) >= TPR ? NOUT * (int)sizeof(T) / TPR : 1; // 16-byte pieces a thread, when QREG
         constexpr bool AHEAD = QREG && WP == 1;
-        constexpr int BATCH = LOADS < 8 ? LOADS : 8; // held at once
-        const int pieces = p.rank * (int)sizeof(T) / 16;
+        constexpr int BATCH = LOADS < 8 || AHEAD ? LOADS : WP == 4 && NOUT >= 32 ? 4 : 8; // held at once
+        const int pieces = rank * (int)sizeof(T) / 16;
         const int srow = threadIdx.x / TPR, sseg = threadIdx.x % TPR;
         u32x4 held[QREG ? BATCH : 1];
         auto request = [&](int p0, int i0) __attribute__((always_inline)) {
             // rows past the end are masked; they only must be numbers
-            const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)(p0 + srow <= kmax ? p0 + srow : kmax) * p.rank) + sseg;
+            const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)(p0 + srow <= kmax ? p0 + srow : kmax) * rank) + sseg;
 #pragma unroll
             for (int i = 0; i < BATCH; ++i)
                 held[i] = src[sseg + (i0 + i) * TPR < pieces ? (i0 + i) * TPR : 0];
         };
         auto put = [&](int buf, int i0) __attribute__((always_inline)) {
-            u32x4 *dst = reinterpret_cast<u32x4 *>(reinterpret_cast<T *>(smem) + (buf * PT + srow) * ld) + sseg;
+            u32x4 *dst = reinterpret_cast<u32x4 *>(reinterpret_cast<T *>(smem) + (buf * PT + srow) * ld);
 #pragma unroll
             for (int i = 0; i < BATCH; ++i)
                 if (sseg + (i0 + i) * TPR < pieces)
-                    dst[(i0 + i) * TPR] = held[i];
+                    dst[(sseg + (i0 + i) * TPR) ^ lat_swizzle(srow)] = held[i];
         };
         if constexpr (AHEAD)
             request(k0, 0);
 
         const int qrow = rb + wr * 16 + c < R ? rb + wr * 16 + c : R - 1;
-        const T *q = static_cast<const T *>(p.q) + ((size_t)p.row0[e] * p.heads + qrow) * p.rank + 8 * g;
+        const T *q = static_cast<const T *>(p.q) + ((size_t)p.row0[e] * p.heads + qrow) * rank + 8 * g;
         V qreg[QREG ? NOUT / 2 : 1];
         if (QREG)
         {
@@ -113,7 +141,7 @@ namespace llamql
         }
         const int limit = rb + wr * 16 + c < R ? pos0 + qrow / p.heads : -1; // newest position this lane's row c sees
         const int tile0 = slice * NOUT + half * NT;                         // the wavefront's first output tile
-        const int out_tiles = (p.rank >> 4) - tile0 < NT ? (p.rank >> 4) - tile0 : NT;
+        const int out_tiles = FULL || (rank >> 4) - tile0 > NT ? NT : (rank >> 4) - tile0;
 
         float m = -INFINITY, l = 0.0f; // of row c; l: this lane's positions only
         f32x4 acc[NT];
@@ -144,34 +172,57 @@ namespace llamql
                 else
                 {
                     const int pos = kt + srow <= kmax ? kt + srow : kmax;
-                    const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)pos * p.rank);
+                    const u32x4 *src = reinterpret_cast<const u32x4 *>(cache + (size_t)pos * rank);
                     u32x4 *dst = reinterpret_cast<u32x4 *>(reinterpret_cast<T *>(smem) + srow * ld);
                     for (int i = sseg; i < pieces; i += TPR)
-                        dst[i] = src[i];
+                        dst[i ^ lat_swizzle(srow)] = src[i];
                 }
             }
             __syncthreads();
 
-            const T *mine = reinterpret_cast<const T *>(smem) + (buf * PT + wp * 32) * ld;
-            const T *keys = mine + (16 * half + c) * ld + 8 * g;
-            f32x4 s[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
+            // (the swizzle of a row of a 16-row block is that of the row in the block)
+            const T *mine = reinterpret_cast<const T *>(smem) + (buf * PT + wp * PG) * ld;
+            const u32x4 *keys = reinterpret_cast<const u32x4 *>(mine + (half * (PG / 2) + c) * ld);
+            const int key_swizzle = lat_swizzle(c);
+            auto key = [&](int block, int ks) __attribute__((always_inline)) {
+                const u32x4 *row = keys + block * (16 * pieces);
+                if constexpr (sizeof(T) == 2)
+                    return __builtin_bit_cast(bf16x8, row[(4 * ks + g) ^ key_swizzle]);
+                else
+                    return __builtin_shufflevector(__builtin_bit_cast(f32x4, row[(8 * ks + 2 * g) ^ key_swizzle]),
+                                                   __builtin_bit_cast(f32x4, row[(8 * ks + 2 * g + 1) ^ key_swizzle]), 0, 1, 2, 3, 4, 5, 6, 7);
+            };
+            f32x4 s[PS][2];
+#pragma unroll
+            for (int b = 0; b < PS; ++b)
+                s[b][0] = s[b][1] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
             if (QREG)
             {
 #pragma unroll
                 for (int ks = 0; ks < NOUT / 2; ++ks)
                     if (ks < ksteps)
-                        s[ks & 1] = O::mma(qreg[ks], O::load(keys + ks * 32), s[ks & 1]);
+                    {
+#pragma unroll
+                        for (int b = 0; b < PS; ++b)
+                            s[b][ks & 1] = O::mma(qreg[ks], key(b, ks), s[b][ks & 1]);
+                    }
             }
             else
                 for (int ks = 0; ks < ksteps; ks += 2) // (the rank is a multiple of 64)
                 {
-                    s[0] = O::mma(O::load(q + ks * 32), O::load(keys + ks * 32), s[0]);
-                    s[1] = O::mma(O::load(q + ks * 32 + 32), O::load(keys + ks * 32 + 32), s[1]);
-                }
-            s[0] = s[0] + s[1];
+                    const V a0 = O::load(q + ks * 32), a1 = O::load(q + ks * 32 + 32);
 #pragma unroll
-            for (int r = 0; r < 4; ++r)
-                s_s[group][(4 * g + r) * SLD + 16 * half + c] = s[0][r];
+                    for (int b = 0; b < PS; ++b)
+                    {
+                        s[b][0] = O::mma(a0, key(b, ks), s[b][0]);
+                        s[b][1] = O::mma(a1, key(b, ks + 1), s[b][1]);
+                    }
+                }
+#pragma unroll
+            for (int b = 0; b < PS; ++b)
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    s_s[group][(4 * g + r) * SLD + half * (PG / 2) + 16 * b + c] = s[b][0][r] + s[b][1][r];
             if constexpr (AHEAD)
             {
                 if (kt + PT < k1)
@@ -183,31 +234,38 @@ namespace llamql
             }
             __syncthreads();
 
-            // row c, positions 8 g .. 8 g + 7 of the group's 32
-            f32x8 w = Operand<float>::load(&s_s[group][c * SLD + 8 * g]);
+            // row c, positions 32 b + 8 g .. + 7 of the group's
+            f32x8 w[PS];
             float mx = m;
 #pragma unroll
-            for (int j = 0; j < 8; ++j)
+            for (int b = 0; b < PS; ++b)
             {
-                w[j] = kt + wp * 32 + 8 * g + j <= limit ? w[j] * p.scale : -INFINITY;
-                mx = fmaxf(mx, w[j]);
+                w[b] = Operand<float>::load(&s_s[group][c * SLD + 32 * b + 8 * g]);
+#pragma unroll
+                for (int j = 0; j < 8; ++j)
+                {
+                    w[b][j] = kt + wp * PG + 32 * b + 8 * g + j <= limit ? w[b][j] * p.scale : -INFINITY;
+                    mx = fmaxf(mx, w[b][j]);
+                }
             }
             mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
             mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
             const float base = mx == -INFINITY ? 0.0f : mx;
             const float alpha = fast_exp(m - base);
-            const bool moved = mx != m;
             m = mx;
             l *= alpha;
+            V wv[PS][PW];
 #pragma unroll
-            for (int j = 0; j < 8; ++j)
+            for (int b = 0; b < PS; ++b)
             {
-                w[j] = fast_exp(w[j] - base);
-                l += w[j];
+#pragma unroll
+                for (int j = 0; j < 8; ++j)
+                {
+                    w[b][j] = fast_exp(w[b][j] - base);
+                    l += w[b][j];
+                }
+                split_pieces<T, PW>(w[b], wv[b]);
             }
-            V wv[PW];
-            split_pieces<T, PW>(w, wv);
-            if (__any(moved)) // most turns move no maximum
             {
                 float a[4];
 #pragma unroll
@@ -221,19 +279,21 @@ namespace llamql
             }
             constexpr int VG = sizeof(T) == 2 ? 4 : 2; // independent products in a row (NT is a multiple)
 #pragma unroll
-            for (int t = 0; t < NT; t += VG)
-                if (t < out_tiles)
-                {
-                    V v[VG];
+            for (int b = 0; b < PS; ++b)
 #pragma unroll
-                    for (int k = 0; k < VG; ++k) // (a tile past the rank: the first one again, its result is not used)
-                        v[k] = load_columns(mine + (tile0 + (t + k < out_tiles ? t + k : 0)) * 16, ld, lane);
+                for (int t = 0; t < NT; t += VG)
+                    if (t < out_tiles)
+                    {
+                        V v[VG];
 #pragma unroll
-                    for (int i = 0; i < PW; ++i)
+                        for (int k = 0; k < VG; ++k) // (tiles past the rank come in fours: none is begun)
+                            v[k] = lat_columns(mine + 32 * b * ld, ld, tile0, t + k, lane);
 #pragma unroll
-                        for (int k = 0; k < VG; ++k)
-                            acc[t + k] = O::mma(wv[i], v[k], acc[t + k]);
-                }
+                        for (int i = 0; i < PW; ++i)
+#pragma unroll
+                            for (int k = 0; k < VG; ++k)
+                                acc[t + k] = O::mma(wv[b][i], v[k], acc[t + k]);
+                    }
             if constexpr (AHEAD)
                 buf ^= 1;
         }
@@ -291,7 +351,7 @@ namespace llamql
             }
             __syncthreads();
             // a wavefront takes every eighth row
-            const int columns = p.rank - slice * NOUT * 16 < NOUT * 16 ? p.rank - slice * NOUT * 16 : NOUT * 16;
+            const int columns = rank - slice * NOUT * 16 < NOUT * 16 ? rank - slice * NOUT * 16 : NOUT * 16;
             for (int row = wave; row < WR * 16 && rb + row < R; row += LAT_THREADS / 64)
                 for (int d = lane * 4; d < columns; d += 256)
                 {
@@ -301,10 +361,10 @@ namespace llamql
                         y = y + *reinterpret_cast<const f32x4 *>(s_o + (w * WR * 16 + row) * OLD + d) * s_f[w * WR * 16 + row];
                     const int col = slice * NOUT * 16 + d;
                     if (p.nsplit == 1)
-                        *reinterpret_cast<t4 *>(static_cast<T *>(p.o) + ((size_t)p.row0[e] * p.heads + rb + row) * p.rank + col) =
+                        *reinterpret_cast<t4 *>(static_cast<T *>(p.o) + ((size_t)p.row0[e] * p.heads + rb + row) * rank + col) =
                             __builtin_convertvector(y, t4);
                     else
-                        *reinterpret_cast<f32x4 *>(p.part_o + (((size_t)ei * p.nsplit + split) * p.rcap + rb + row) * p.rank + col) = y;
+                        *reinterpret_cast<f32x4 *>(p.part_o + (((size_t)ei * p.nsplit + split) * p.rcap + rb + row) * rank + col) = y;
                 }
             return;
         }
@@ -322,9 +382,9 @@ namespace llamql
                 {
                     const int col = (tile0 + t) * 16 + c;
                     if (p.nsplit == 1)
-                        static_cast<T *>(p.o)[((size_t)p.row0[e] * p.heads + row) * p.rank + col] = (T)(acc[t][r] * inv);
+                        static_cast<T *>(p.o)[((size_t)p.row0[e] * p.heads + row) * rank + col] = (T)(acc[t][r] * inv);
                     else
-                        p.part_o[at * p.rank + col] = acc[t][r];
+                        p.part_o[at * rank + col] = acc[t][r];
                 }
         }
         if (p.nsplit > 1 && half == 0 && g == 0 && slice == 0 && rb + wr * 16 + c < R)
@@ -421,31 +481,42 @@ namespace llamql
 
     namespace
     {
-        template <typename T, int NOUT, bool QREG, int WR>
+        template <typename T, int NOUT, bool QREG, bool FULL, int WR>
         bool latent_launch(const char *fn, const LatentArgs &p, int row_blocks, int n, hipStream_t st)
         {
             static LdsGrant grant;
             constexpr int WP = 4 / WR;
-            size_t lds = (size_t)32 * WP * (p.rank + LAT_PAD / sizeof(T)) * sizeof(T) * (QREG && WP == 1 ? 2 : 1);
+            size_t lds = (size_t)lat_group(NOUT, QREG, WR) * WP * (QREG && WP == 1 ? 2 : 1) * p.rank * sizeof(T);
             const size_t merge = WP > 1 ? (size_t)64 * (NOUT * 16 + 4) * 4 : 0;
             lds = lds > merge ? lds : merge;
-            constexpr size_t most = 150 * 1024;
+            constexpr size_t most = 142 * 1024; // beside the scores
             if (lds > most)
                 return fail(fn, "rank=%d does not fit the LDS", p.rank);
-            if (lds > 48 * 1024 && allow_lds(grant, reinterpret_cast<const void *>(&latent_attention_kernel<T, NOUT, QREG, WR>), most) != hipSuccess)
+            if (lds > 48 * 1024 && allow_lds(grant, reinterpret_cast<const void *>(&latent_attention_kernel<T, NOUT, QREG, FULL, WR>), most) != hipSuccess)
                 return fail(fn, "cannot reserve %zu bytes of LDS", lds);
-            hipLaunchKernelGGL((latent_attention_kernel<T, NOUT, QREG, WR>), dim3(row_blocks, p.nsplit, n * p.slices),
+            hipLaunchKernelGGL((latent_attention_kernel<T, NOUT, QREG, FULL, WR>), dim3(row_blocks, p.nsplit, n * p.slices),
                                dim3(LAT_THREADS), lds, st, p);
             return launched(fn);
         }
+        template <typename T, int NOUT, bool QREG, bool FULL>
+        bool latent_stretches(const char *fn, const LatentArgs &p, int wr, int row_blocks, int n, hipStream_t st)
+        {
+            if (wr == 1)
+                return latent_launch<T, NOUT, QREG, FULL, 1>(fn, p, row_blocks, n, st);
+            if (wr == 2)
+                return latent_launch<T, NOUT, QREG, FULL, 2>(fn, p, row_blocks, n, st);
+            return latent_launch<T, NOUT, QREG, FULL, 4>(fn, p, row_blocks, n, st);
+        }
+
         template <typename T, int NOUT, bool QREG>
         bool latent_rows(const char *fn, const LatentArgs &p, int wr, int row_blocks, int n, hipStream_t st)
         {
-            if (wr == 1)
-                return latent_launch<T, NOUT, QREG, 1>(fn, p, row_blocks, n, st);
-            if (wr == 2)
-                return latent_launch<T, NOUT, QREG, 2>(fn, p, row_blocks, n, st);
-            return latent_launch<T, NOUT, QREG, 4>(fn, p, row_blocks, n, st);
+            if constexpr (QREG && sizeof(T) == 2)
+            {
+                if (p.rank == 16 * NOUT)
+                    return latent_stretches<T, NOUT, QREG, true>(fn, p, wr, row_blocks, n, st);
+            }
+            return latent_stretches<T, NOUT, QREG, false>(fn, p, wr, row_blocks, n, st);
         }
 
         // how a call is cut up: wavefronts per row group and stretches of the sequence
@@ -461,11 +532,11 @@ namespace llamql
             while (pl.wr < 4)
             {
                 const int wp = 4 / pl.wr;
-                if ((size_t)32 * wp * (rank + LAT_PAD / elem) * elem <= 140 * 1024)
+                if ((size_t)32 * wp * rank * elem <= 140 * 1024)
                     break;
                 pl.wr *= 2;
             }
-            const int pt = 32 * (4 / pl.wr);
+            const int pt = pl.wr == 4 ? 64 : 32 * (4 / pl.wr);
             pl.row_blocks = ceil_div(R, 16 * pl.wr);
             int nsplit = ceil_div(LAT_TARGET, pl.row_blocks * n);
             const int most = ceil_div(max_len, pt > LAT_MIN_STRETCH ? pt : LAT_MIN_STRETCH);
