@@ -260,10 +260,11 @@ namespace llamql
     }
 
     // ---- prompts: the walk over the chunks ----------------------------------------------------------
-    // Workgroup = up to four wavefronts of 16 columns each, of one head.  DT: 16-row tiles of S (dim <= 16 DT).
+    // Workgroup = up to four wavefronts of 16 columns each, of one head.  DT: 16-row tiles of S (dim <= 16 DT); FULL:
+    // dim is 16 DT exactly, so that no product hangs on a condition.
     // What the next chunk needs from memory (q and k for the LDS, this column's values, the products) is
     // requested before the matrix work of the current one.
-    template <typename T, int LC, int DT>
+    template <typename T, int LC, int DT, bool FULL>
     __global__ void __launch_bounds__(256)
         memory_chunk_kernel(MemoryArgs p)
     {
@@ -280,15 +281,16 @@ namespace llamql
         const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
         const int h = blockIdx.y, e = p.entry;
         const int ntok = p.ntok[e], slot = p.slot[e], row0 = p.row0[e];
-        const int ldv = p.vdim + 16, ld = p.dim + LPAD;
+        const int dim = FULL ? 16 * DT : p.dim;
+        const int ldv = p.vdim + 16, ld = dim + LPAD;
         const int col = (blockIdx.x * 4 + wave) * 16 + c;
         const bool live = (blockIdx.x * 4 + wave) * 16 < ldv; // of the wavefront
         const bool ones = (blockIdx.x * 4 + wave) * 16 == p.vdim;
         T *sq = reinterpret_cast<T *>(smem), *sk = sq + LC * ld;
-        const int dtiles = p.dim >> 4;
+        const int dtiles = FULL ? DT : dim >> 4;
 
         f32x4 S[DT];
-        float *state = p.state + ((size_t)slot * p.heads + h) * p.dim * ldv + (live ? col : 0);
+        float *state = p.state + ((size_t)slot * p.heads + h) * dim * ldv + (live ? col : 0);
         const bool fresh = p.pos[e] == 0;
 #pragma unroll
         for (int t = 0; t < DT; ++t)
@@ -302,9 +304,9 @@ namespace llamql
             }
         }
 
-        const int srow = threadIdx.x / TPR, sseg = threadIdx.x % TPR, pieces = p.dim * (int)sizeof(T) / 16;
-        const T *qrows = static_cast<const T *>(p.qk) + (size_t)h * p.qk_rows * p.dim;
-        const T *krows = qrows + (size_t)p.heads * p.qk_rows * p.dim;
+        const int srow = threadIdx.x / TPR, sseg = threadIdx.x % TPR, pieces = dim * (int)sizeof(T) / 16;
+        const T *qrows = static_cast<const T *>(p.qk) + (size_t)h * p.qk_rows * dim;
+        const T *krows = qrows + (size_t)p.heads * p.qk_rows * dim;
         u32x4 hq[AHEAD ? LOADS : 1], hk[AHEAD ? LOADS : 1];
         f32x8 hv[LC / 32];
         double h_ga = 0.0, h_a = 0.0, h_end = 0.0;
@@ -315,8 +317,8 @@ namespace llamql
             if constexpr (AHEAD)
             {
                 // (the product kernel wrote whole chunks: rows past the portion repeat its last one)
-                const u32x4 *q = reinterpret_cast<const u32x4 *>(qrows + (size_t)(t0 + srow) * p.dim) + sseg;
-                const u32x4 *k = reinterpret_cast<const u32x4 *>(krows + (size_t)(t0 + srow) * p.dim) + sseg;
+                const u32x4 *q = reinterpret_cast<const u32x4 *>(qrows + (size_t)(t0 + srow) * dim) + sseg;
+                const u32x4 *k = reinterpret_cast<const u32x4 *>(krows + (size_t)(t0 + srow) * dim) + sseg;
 #pragma unroll
                 for (int i = 0; i < LOADS; ++i)
                 {
@@ -339,7 +341,7 @@ namespace llamql
                 {
                     const int tt = 32 * s + 8 * g + j;
                     hv[s][j] = ones || !live ? 0.0f
-                                             : p.proj[(size_t)(r0 + (tt < n ? tt : n - 1)) * p.ldp + (size_t)p.heads * 2 * p.dim + h * p.vdim + col];
+                                             : p.proj[(size_t)(r0 + (tt < n ? tt : n - 1)) * p.ldp + (size_t)p.heads * 2 * dim + h * p.vdim + col];
                 }
         };
         request(0);
@@ -371,8 +373,8 @@ namespace llamql
                 }
                 else
                 {
-                    const u32x4 *q = reinterpret_cast<const u32x4 *>(qrows + (size_t)(t0 + srow) * p.dim) + sseg;
-                    const u32x4 *k = reinterpret_cast<const u32x4 *>(krows + (size_t)(t0 + srow) * p.dim) + sseg;
+                    const u32x4 *q = reinterpret_cast<const u32x4 *>(qrows + (size_t)(t0 + srow) * dim) + sseg;
+                    const u32x4 *k = reinterpret_cast<const u32x4 *>(krows + (size_t)(t0 + srow) * dim) + sseg;
 #pragma unroll 4
                     for (int i = 0; sseg + i < pieces; i += TPR)
                     {
@@ -643,15 +645,25 @@ namespace llamql
             p.qk = s + at.qk, p.qk_rows = rows;
         }
 
-        template <typename T, int LC, int DT>
-        bool chunk_launch(const char *fn, const MemoryArgs &p, hipStream_t st)
+        template <typename T, int LC, int DT, bool FULL>
+        bool chunk_launch_as(const char *fn, const MemoryArgs &p, hipStream_t st)
         {
             static LdsGrant grant;
             const size_t lds = (size_t)2 * LC * (p.dim + 16 / sizeof(T)) * sizeof(T);
-            if (lds > 48 * 1024 && allow_lds(grant, reinterpret_cast<const void *>(&memory_chunk_kernel<T, LC, DT>), 140 * 1024) != hipSuccess)
+            if (lds > 48 * 1024 && allow_lds(grant, reinterpret_cast<const void *>(&memory_chunk_kernel<T, LC, DT, FULL>), 140 * 1024) != hipSuccess)
                 return fail(fn, "cannot reserve %zu bytes of LDS", lds);
-            hipLaunchKernelGGL((memory_chunk_kernel<T, LC, DT>), dim3(ceil_div(p.vdim + 16, 64), p.heads), dim3(256), lds, st, p);
+            hipLaunchKernelGGL((memory_chunk_kernel<T, LC, DT, FULL>), dim3(ceil_div(p.vdim + 16, 64), p.heads), dim3(256), lds, st, p);
             return launched(fn);
+        }
+        template <typename T, int LC, int DT>
+        bool chunk_launch(const char *fn, const MemoryArgs &p, hipStream_t st)
+        {
+            if constexpr (sizeof(T) == 2)
+            {
+                if (p.dim == 16 * DT)
+                    return chunk_launch_as<T, LC, DT, true>(fn, p, st);
+            }
+            return chunk_launch_as<T, LC, DT, false>(fn, p, st);
         }
         template <typename T, int LC>
         bool prefill_run(const char *fn, const MemoryArgs &p, int ntok, hipStream_t st)

@@ -62,12 +62,16 @@ MECHANISMS = {
     "latent 20 heads": [sm.latent(heads=20, dim=12, vdim=4, q_rank=64, kv_rank=64)],
     "latent rank 200": [sm.latent(heads=18, kv_rank=200)],
     "latent rank 330": [sm.latent(kv_rank=330)],
+    "latent rank 512": [sm.latent(heads=4, kv_rank=512)],
+    "latent rank 150": [sm.latent(heads=9, kv_rank=150)],
     "latent rank 600": [sm.latent(heads=5, kv_rank=600)],
     "latent shared": [sm.latent(), sm.latent(kv_from=0, heads=7, dim=20, vdim=70, q_rank=90, scale=0.7)],
     "mlstm": [sm.mlstm()],
     "mlstm one head": [sm.mlstm(heads=1, dim=16, vdim=88, gate_cap=2.5)],
     "mlstm dim 130": [sm.mlstm(heads=2, dim=130, vdim=33)],
     "mlstm dim 300": [sm.mlstm(heads=2, dim=300, vdim=150, gate_cap=15.0)],
+    "mlstm dim 256": [sm.mlstm(heads=1, dim=256, vdim=64, gate_cap=30.0)],
+    "mlstm dim 512": [sm.mlstm(heads=1, dim=500, vdim=96)],
     "dense": [sm.mlstm(heads=1, dim=8, vdim=8, mlp=sm.dense())],
     "experts": [sm.mlstm(heads=1, dim=8, vdim=8, mlp=sm.moe())],
     "experts shared": [sm.latent(mlp=sm.moe(ff=40, experts=12, top=5, shared=136))],
@@ -346,3 +350,27 @@ def test_programs_run_a_model_from_its_folder(tmp_path, whole):
     output = [int(x) for x in p.stdout.strip().split(",")]
     logits = so.kogilix(WHOLE, t.plain(), tokens[:10] + output)[9:-1]
     assert output == logits.argmax(axis=1).tolist()
+
+
+def test_the_dense_family_behind_the_same_engine(tmp_path, dev):
+    """The quantized dense decoder served by the scheduler: the tokens of its own step driver fed by hand."""
+    from llaminar_amd import decoder, models
+
+    (tmp_path / "config.json").write_text(json.dumps({"architecture": "DenseQ4K", "hidden": 512, "n_heads": 4, "n_kv": 2,
+                                                      "ffn": 768, "vocab": 1000, "n_layers": 2, "seed": 3}))
+    prompts = [[5, 9, 11], [7], [100, 200, 300, 400, 500, 600]]
+    runner = models.load_model(tmp_path, slots=2, cap=40)
+    got = Engine(runner, portion=2).generate(prompts, 6)
+    runner.close()
+    for prompt, output in zip(prompts, got):
+        dec = decoder.DenseDecoder(decoder.Shape(512, 4, 2, 128, 768, 1000, 2), 2, 64, dev, seed=3)
+        want, tokens = [], list(prompt)
+        for n in range(len(prompt) + 5):
+            dec.set_state([tokens[n], 0], [n, 0])
+            dec.step()
+            chosen = int(dec.buffer("ids").cpu()[0])
+            if n >= len(prompt) - 1:
+                want.append(chosen)
+                tokens.append(chosen)
+        dec.close()
+        assert output == want
