@@ -5,12 +5,12 @@
 // entry, all against the same keys.  A workgroup takes 16 WR rows and a stretch of the sequence,
 // and walks it 32 WP positions at a time (WR * WP = 4 groups of two wavefronts), the cache rows
 // staged once in LDS:
-//   scores  S[row][p] = sum_d q[row][d] c[p][d]   second operand: c rows as they lie; each wavefront
-//                                                  of a pair takes 16 of the group's 32 positions
-//   output  O[row][d] = sum_p w[row][p] c[p][d]   second operand: c columns (transposing LDS read);
+//   scores  S[p][row] = sum_d c[p][d] q[row][d]   first operand: c rows as they lie; each wavefront
+//                                                  of a pair takes half of the group's positions
+//   output  O[d][row] = sum_p c[p][d] w[row][p]   first operand: c columns (transposing LDS read);
 //                                                  each takes half of the columns
-// In between the scores pass through LDS, where both read them as first operand of the output
-// product and keep the running maximum and sum of their rows.  Softmax in 32-bit; for bf16 the
+// so that a lane's results belong to one row.  In between the scores pass through LDS, where both
+// wavefronts read them as second operand of the output product and keep the running maximum and sum of their rows.  Softmax in 32-bit; for bf16 the
 // weights enter the product as two bf16 pieces.  With WP > 1 the groups of a row block split the
 // positions and merge through LDS; with several stretches per row block a second kernel merges those.
 #include "seq_common.h"
@@ -204,7 +204,7 @@ namespace llamql
                     {
 #pragma unroll
                         for (int b = 0; b < PS; ++b)
-                            s[b][ks & 1] = O::mma(qreg[ks], key(b, ks), s[b][ks & 1]);
+                            s[b][ks & 1] = O::mma(key(b, ks), qreg[ks], s[b][ks & 1]);
                     }
             }
             else
@@ -214,15 +214,13 @@ namespace llamql
 #pragma unroll
                     for (int b = 0; b < PS; ++b)
                     {
-                        s[b][0] = O::mma(a0, key(b, ks), s[b][0]);
-                        s[b][1] = O::mma(a1, key(b, ks + 1), s[b][1]);
+                        s[b][0] = O::mma(key(b, ks), a0, s[b][0]);
+                        s[b][1] = O::mma(key(b, ks + 1), a1, s[b][1]);
                     }
                 }
 #pragma unroll
-            for (int b = 0; b < PS; ++b)
-#pragma unroll
-                for (int r = 0; r < 4; ++r)
-                    s_s[group][(4 * g + r) * SLD + half * (PG / 2) + 16 * b + c] = s[b][0][r] + s[b][1][r];
+            for (int b = 0; b < PS; ++b) // lane: row c, positions 4 g .. 4 g + 3
+                *reinterpret_cast<f32x4 *>(&s_s[group][c * SLD + half * (PG / 2) + 16 * b + 4 * g]) = s[b][0] + s[b][1];
             if constexpr (AHEAD)
             {
                 if (kt + PT < k1)
@@ -266,17 +264,9 @@ namespace llamql
                 }
                 split_pieces<T, PW>(w[b], wv[b]);
             }
-            {
-                float a[4];
 #pragma unroll
-                for (int r = 0; r < 4; ++r)
-                    a[r] = __shfl(alpha, 4 * g + r, 64);
-#pragma unroll
-                for (int t = 0; t < NT; ++t)
-#pragma unroll
-                    for (int r = 0; r < 4; ++r)
-                        acc[t][r] *= a[r];
-            }
+            for (int t = 0; t < NT; ++t)
+                acc[t] = acc[t] * alpha;
             constexpr int VG = sizeof(T) == 2 ? 4 : 2; // independent products in a row (NT is a multiple)
 #pragma unroll
             for (int b = 0; b < PS; ++b)
@@ -292,7 +282,7 @@ namespace llamql
                         for (int i = 0; i < PW; ++i)
 #pragma unroll
                             for (int k = 0; k < VG; ++k)
-                                acc[t + k] = O::mma(wv[b][i], v[k], acc[t + k]);
+                                acc[t + k] = O::mma(v[k], wv[b][i], acc[t + k]);
                     }
             if constexpr (AHEAD)
                 buf ^= 1;
@@ -310,11 +300,7 @@ namespace llamql
 #pragma unroll
             for (int t = 0; t < NT; ++t)
                 if (t < out_tiles)
-                {
-#pragma unroll
-                    for (int r = 0; r < 4; ++r)
-                        s_o[(group * 16 + 4 * g + r) * OLD + (half * NT + t) * 16 + c] = acc[t][r];
-                }
+                    *reinterpret_cast<f32x4 *>(s_o + (group * 16 + c) * OLD + (half * NT + t) * 16 + 4 * g) = acc[t];
             if (half == 0 && g == 0)
             {
                 s_ml[(group * 16 + c) * 2] = m;
@@ -368,28 +354,24 @@ namespace llamql
                 }
             return;
         }
+        const int row = rb + wr * 16 + c;
+        if (row >= R)
+            return;
+        const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + row;
+        const float inv = 1.0f / l;
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
+        for (int t = 0; t < NT; ++t)
+            if (t < out_tiles)
+            {
+                const int col = (tile0 + t) * 16 + 4 * g;
+                if (p.nsplit == 1)
+                    *reinterpret_cast<t4 *>(static_cast<T *>(p.o) + ((size_t)p.row0[e] * p.heads + row) * rank + col) =
+                        __builtin_convertvector(acc[t] * inv, t4);
+                else
+                    *reinterpret_cast<f32x4 *>(p.part_o + at * rank + col) = acc[t];
+            }
+        if (p.nsplit > 1 && half == 0 && g == 0 && slice == 0)
         {
-            const int row = rb + wr * 16 + 4 * g + r;
-            const float inv = 1.0f / __shfl(l, 4 * g + r, 64);
-            if (row >= R)
-                continue;
-            const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + row;
-#pragma unroll
-            for (int t = 0; t < NT; ++t)
-                if (t < out_tiles)
-                {
-                    const int col = (tile0 + t) * 16 + c;
-                    if (p.nsplit == 1)
-                        static_cast<T *>(p.o)[((size_t)p.row0[e] * p.heads + row) * rank + col] = (T)(acc[t][r] * inv);
-                    else
-                        p.part_o[at * rank + col] = acc[t][r];
-                }
-        }
-        if (p.nsplit > 1 && half == 0 && g == 0 && slice == 0 && rb + wr * 16 + c < R)
-        {
-            const size_t at = ((size_t)ei * p.nsplit + split) * p.rcap + rb + wr * 16 + c;
             p.part_ml[at * 2] = m;
             p.part_ml[at * 2 + 1] = l;
         }
@@ -536,7 +518,7 @@ namespace llamql
                     break;
                 pl.wr *= 2;
             }
-            const int pt = pl.wr == 4 ? 64 : 32 * (4 / pl.wr);
+            const int pt = pl.wr == 4 ? (rank > 256 ? 32 : 64) : 32 * (4 / pl.wr);
             pl.row_blocks = ceil_div(R, 16 * pl.wr);
             int nsplit = ceil_div(LAT_TARGET, pl.row_blocks * n);
             const int most = ceil_div(max_len, pt > LAT_MIN_STRETCH ? pt : LAT_MIN_STRETCH);
