@@ -64,12 +64,33 @@ namespace llamql
         int ldx;
         int *ids;       // [M][top]
         float *weights; // [M][top + 1]: of the chosen experts, then of the shared one
+        bool routed;    // few rows: ids and weights are there already
         void *act;      // T: few rows [M][top * ff + shared_ff], many rows [M * top][ff] then [M][shared_ff]
     };
 
-    // Few rows.  Workgroup = 16 outputs of one expert of one token.  All workgroups choose the
-    // token's experts for themselves from the logits; the first of a token records the choice for
-    // the down projections.
+    // A wavefront per token chooses its experts.
+    __global__ void __launch_bounds__(ROW_THREADS)
+        expert_route_kernel(ExpertArgs p, int M)
+    {
+        const int lane = threadIdx.x & 63, m = blockIdx.x * (ROW_THREADS / 64) + (threadIdx.x >> 6);
+        if (m >= M)
+            return;
+        const float *z = p.logits + (size_t)m * p.ldz;
+        int id;
+        float weight;
+        route_wave(z, p.experts, p.top, lane, id, weight);
+        if (lane < p.top)
+        {
+            p.ids[m * p.top + lane] = id;
+            p.weights[m * (p.top + 1) + lane] = weight;
+        }
+        if (lane == 0 && p.shared_ff)
+            p.weights[m * (p.top + 1) + p.top] = sigmoidf(z[p.experts]);
+    }
+
+    // Few rows.  Workgroup = 16 outputs of one expert of one token.  With a single row all workgroups
+    // choose the token's experts for themselves from the logits, and the first records the choice for
+    // the down projections; with more, a launch before has chosen.
     constexpr int EXPERT_WAVES = 8;
     template <typename T>
     __global__ void __launch_bounds__(EXPERT_WAVES * 64)
@@ -89,8 +110,11 @@ namespace llamql
         {
             if (tile * 16 >= p.ff)
                 return;
-            route_wave(z, p.experts, p.top, lane, id, weight);
-            if (tile == 0 && job == 0 && wave == 0)
+            if (p.routed)
+                id = p.ids[m * p.top + job];
+            else
+                route_wave(z, p.experts, p.top, lane, id, weight);
+            if (!p.routed && tile == 0 && job == 0 && wave == 0)
             {
                 if (lane < p.top)
                 {
@@ -216,27 +240,8 @@ namespace llamql
         }
     }
 
-    // Many rows: a wavefront per token chooses the experts ...
-    __global__ void __launch_bounds__(ROW_THREADS)
-        expert_route_kernel(ExpertArgs p, int M)
-    {
-        const int lane = threadIdx.x & 63, m = blockIdx.x * (ROW_THREADS / 64) + (threadIdx.x >> 6);
-        if (m >= M)
-            return;
-        const float *z = p.logits + (size_t)m * p.ldz;
-        int id;
-        float weight;
-        route_wave(z, p.experts, p.top, lane, id, weight);
-        if (lane < p.top)
-        {
-            p.ids[m * p.top + lane] = id;
-            p.weights[m * (p.top + 1) + lane] = weight;
-        }
-        if (lane == 0 && p.shared_ff)
-            p.weights[m * (p.top + 1) + p.top] = sigmoidf(z[p.experts]);
-    }
-
-    // ... the (token, choice) pairs are put in order of their expert, each expert's in the order of
+    // Many rows: after the choice of experts
+    // the (token, choice) pairs are put in order of their expert, each expert's in the order of
     // the tokens: one workgroup per expert counts the pairs of lower experts and places its own
     constexpr int GROUP_THREADS = 1024;
     __global__ void __launch_bounds__(GROUP_THREADS)
@@ -288,7 +293,7 @@ namespace llamql
         }
     }
 
-    // ... and the experts' outputs are summed in the order of the choice
+    // and the experts' outputs are summed in the order of the choice
     __global__ void __launch_bounds__(ROW_THREADS)
         expert_combine_kernel(ExpertArgs p, const float *__restrict__ pair_out, const float *__restrict__ shared_out,
                               const int *__restrict__ place)
@@ -343,6 +348,13 @@ namespace llamql
             p.ids = reinterpret_cast<int *>(scratch + at.ids);
             p.weights = reinterpret_cast<float *>(scratch + at.weights);
             p.act = scratch + at.act;
+            if (M > 1)
+            {
+                hipLaunchKernelGGL(expert_route_kernel, dim3(ceil_div(M, ROW_THREADS / 64)), dim3(ROW_THREADS), 0, st, p, M);
+                if (!launched(fn))
+                    return false;
+                p.routed = true;
+            }
             if (M <= SMALL_M)
             {
                 const int widest = p.shared_ff > p.ff ? p.shared_ff : p.ff;
@@ -357,9 +369,6 @@ namespace llamql
             int *place = reinterpret_cast<int *>(scratch + at.place);
             float *pair_out = reinterpret_cast<float *>(scratch + at.pair_out);
             float *shared_out = reinterpret_cast<float *>(scratch + at.shared_out);
-            hipLaunchKernelGGL(expert_route_kernel, dim3(ceil_div(M, ROW_THREADS / 64)), dim3(ROW_THREADS), 0, st, p, M);
-            if (!launched(fn))
-                return false;
             hipLaunchKernelGGL(expert_group_kernel, dim3(p.experts), dim3(GROUP_THREADS), 0, st, p.ids, M * p.top, p.experts,
                                offset, order, place);
             if (!launched(fn))

@@ -135,6 +135,29 @@ namespace llamql
     constexpr int ROUTE_MAX = 16; // up to 1024 experts
     __device__ __forceinline__ void route_wave(const float *z, int n, int top, int lane, int &id, float &weight)
     {
+        if (n <= 64)
+        {
+            // an expert a lane: its place is the number of experts ahead of it
+            const float v = lane < n ? z[lane] : -INFINITY;
+            int place = 0;
+            for (int e = 0; e < n; ++e)
+            {
+                const float o = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), e));
+                place += o > v || (o == v && e < lane) ? 1 : 0;
+            }
+            id = 0;
+            for (int t = 0; t < top; ++t)
+            {
+                const unsigned long long at = __ballot(place == t && lane < n);
+                const int who = at ? __builtin_ctzll(at) : t; // (none: only with logits that are not numbers)
+                if (lane == t)
+                    id = who;
+            }
+            const float mine = __shfl(v, id, WAVE64), first = __shfl(v, __builtin_amdgcn_readfirstlane(id), WAVE64);
+            const float e = lane < top ? expf(mine - first) : 0.0f;
+            weight = e / wave_sum64(e);
+            return;
+        }
         float v[ROUTE_MAX];
 #pragma unroll
         for (int i = 0; i < ROUTE_MAX; ++i)
