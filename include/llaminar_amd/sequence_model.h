@@ -1,14 +1,17 @@
 /* Host-side driver of decoder-only models whose layers are chosen one by one: each layer has a
- * token mixer (latent attention or a matrix-memory recurrence) and a feed-forward (gated, routed
- * experts, or none), pre-norm, over plain bf16 weights.  C ABI over an opaque handle, exported by
+ * token mixer (latent or grouped-query attention, a matrix-memory or a delta-rule recurrence) and a
+ * feed-forward (gated, routed experts, or none), pre-norm, over plain bf16 weights.  C ABI over an opaque handle, exported by
  * libllaminar_seq.so together with the operators of seq_api.h, which do all the arithmetic.
  *
- *   x = embed[ids]
+ *   x = embed_scale embed[ids] (+ a row per pair of neighbouring ids)
  *   per layer:  x += mixer(rms(x) * norm1);  x += ffn(rms(x) * norm2)
+ *   or, for a parallel layer:  x += mixer(rms(x) * norm1) + ffn(rms(x) * norm2), both of the same x
  *   logits = head (rms(x) * final_norm)
  *
  * The handle owns the sequences' state: `slots` sequences of up to `cap` tokens, per latent layer
- * a cache [slots][cap][rank] (a layer with kv_from reads that layer's), per memory layer fp32 state.
+ * a cache [slots][cap][rank], per grouped-query attention layer a ring of keys and values, long enough for
+ * what the masks of the layers that read it let them see (a layer with kv_from reads that layer's), per memory
+ * or delta layer fp32 state, and the ids themselves where pairs of them are embedded.
  * A sequence starts afresh when an entry names its slot with position 0; nothing has to be cleared.
  *
  * llam_seqm_forward runs one step: any mixture of portions of prompts and single tokens, at most
@@ -27,8 +30,14 @@
 extern "C" {
 #endif
 
-enum { LLAM_MIXER_LATENT_ATTENTION = 1, LLAM_MIXER_MATRIX_MEMORY = 2 };
-enum { LLAM_FFN_NONE = 0, LLAM_FFN_GATED = 1, LLAM_FFN_EXPERTS = 2 };
+enum
+{
+    LLAM_MIXER_LATENT_ATTENTION = 1,
+    LLAM_MIXER_MATRIX_MEMORY = 2,
+    LLAM_MIXER_ATTENTION = 3, /* grouped-query, rotary */
+    LLAM_MIXER_DELTA = 4
+};
+enum { LLAM_FFN_NONE = 0, LLAM_FFN_GATED = 1, LLAM_FFN_EXPERTS = 2, LLAM_FFN_GATED_CLAMP = 3 };
 
 typedef struct
 {
@@ -39,7 +48,7 @@ typedef struct
     int device_id;
 } llam_seqm_config;
 
-/* P(n) = n rounded up to a multiple of 64, H = heads.  Matrices in the tiles of seq_api.h,
+/* P(n) = n rounded up to a multiple of 64, A(n) to 64, 128 or 256, H = heads, G = kv_heads.  Matrices in the tiles of seq_api.h,
  * [rows x columns] padded with zeros; per-head blocks are padded per head.  Vectors fp32, padded
  * with zeros like the columns they belong to.  All device memory, owned by the caller. */
 typedef struct
@@ -50,9 +59,13 @@ typedef struct
     /* latent attention: [P(q_rank) (+ P(kv_rank)) x P(width)]: query latent, then key/value latent
      * (absent with kv_from >= 0).
      * matrix memory: [2 H P(dim) + 2 H P(vdim) + 2 H, rounded up to 16, x P(width)]: q, k, v, output
-     * gate, input gate, forget gate */
+     * gate, input gate, forget gate
+     * attention: [H A(dim) (+ G A(dim) + G A(vdim)), x P(width)]: q (k, v absent with kv_from >= 0)
+     * delta: [2 G P(dim) + 2 H P(vdim) + 2 H, rounded up to 16, x P(width)]: q, k, v, output gate, b, a */
     const void *w_in;
-    const void *w_out; /* [P(width) x H P(vdim)] */
+    /* [P(width) x H P(vdim)], attention: [P(width) x H A(vdim)]; of a parallel layer with a feed-forward
+     * followed by that one's down projection, [P(width) x (H P(vdim) + P(ff))] */
+    const void *w_out;
     /* latent attention */
     int q_rank, kv_rank, kv_from; /* kv_from: the layer whose cache is read, or -1 */
     float scale;
@@ -63,10 +76,20 @@ typedef struct
     /* matrix memory */
     float gate_cap;
     const float *gate_bias; /* [2][H]: input gate, forget gate */
-    const float *head_norm; /* [H][P(vdim)] */
+    const float *head_norm; /* [H][P(vdim)]; delta: [P(vdim)] */
+    /* attention, delta */
+    int kv_heads;
+    /* attention; turns: [rot_dims / 2], revolutions per position; chunk 0: no mask */
+    int rot_dims, chunk;
+    const double *turns;
+    /* delta; conv: [taps][2 G P(dim) + H P(vdim)]; a_log, dt_bias: [H] */
+    int taps;
+    const float *conv, *a_log, *dt_bias;
     /* feed-forward */
+    int parallel; /* with gated feed-forwards; w_down is then part of w_out */
     int ffn;
     const float *norm2;
+    float limit;          /* gated with clamps */
     int ff;               /* gated: its width; experts: an expert's */
     const void *w_up;     /* gated: [2 P(ff) x P(width)], 16-row tiles of gate and up alternating;
                              experts: `experts` matrices [P(ff) x P(width)] */
@@ -82,6 +105,10 @@ typedef struct
     const void *embed;       /* bf16 [vocab][width], row-major */
     const float *final_norm; /* [P(width)] */
     const void *head;        /* [vocab rounded up to 16 x P(width)] */
+    float embed_scale;
+    const void *pairs; /* bf16 [buckets + 1][width], or NULL; see llam_seq_embed */
+    int buckets;
+    long mul_prev, mul_cur;
 } llam_seqm_globals;
 
 void *llam_seqm_create(const llam_seqm_config *cfg);

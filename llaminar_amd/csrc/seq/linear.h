@@ -19,6 +19,7 @@ namespace llamql
         int M, N, K;
         int lda, ldy;
         int out; // LLAM_SEQ_OUT_*
+        float limit;
         long a_stride, w_stride, y_stride;
         // rows in groups (routed experts): group z has the rows group_offset[z] .. group_offset[z + 1] - 1
         // of y; row r reads a[row_source ? row_source[r] / source_div : r]
@@ -30,6 +31,7 @@ namespace llamql
     constexpr int SMALL_M = 16;         // most rows of the row-at-a-time kernel: one operand of the matrix unit
     constexpr int NORM_FUSE_MAX = 8192; // most values (rows x columns) every workgroup norms for itself
 
+    __host__ __device__ inline bool is_gated(int out) { return out == LLAM_SEQ_OUT_GATED || out == LLAM_SEQ_OUT_GATED_CLAMP; }
     bool linear_small(const char *fn, const LinearArgs &a, int batch, int dtype, hipStream_t st);
     bool linear_tiled(const char *fn, const LinearArgs &a, int batch, int dtype, hipStream_t st);
 
@@ -70,9 +72,19 @@ namespace llamql
         }
     }
 
-    __device__ __forceinline__ f32x4 gated4(f32x4 gate, f32x4 up)
+    __device__ __forceinline__ f32x4 gated4(const LinearArgs &p, f32x4 gate, f32x4 up)
     {
         f32x4 v;
+        if (p.out == LLAM_SEQ_OUT_GATED_CLAMP)
+        {
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+            {
+                const float a = fminf(gate[r], p.limit), u = fminf(fmaxf(up[r], -p.limit), p.limit);
+                v[r] = a * sigmoidf(1.702f * a) * (u + 1.0f);
+            }
+            return v;
+        }
 #pragma unroll
         for (int r = 0; r < 4; ++r)
             v[r] = gelu_tanh(gate[r]) * up[r];

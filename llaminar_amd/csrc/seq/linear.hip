@@ -10,12 +10,11 @@
 namespace llamql
 {
     // ---- up to 16 rows ------------------------------------------------------------------------
-    // RT tiles of W per workgroup (2 for a gate tile beside its up tile), NW wavefronts, U k-steps
+    // RT tiles of W per workgroup (2 for a gate tile beside its up tile, or to share the rows), NW wavefronts, U k-steps
     // in flight per wavefront.  NORM: A is fp32, normed by the workgroup into LDS (as T) while the
     // first weights are on their way.
     template <typename T, int NW, int RT, bool NORM>
-    __global__ void __launch_bounds__(NW * 64)
-        linear_small_kernel(LinearArgs p)
+    __device__ __forceinline__ void linear_small_tile(const LinearArgs &p, int block)
     {
         using O = Operand<T>;
         using V = typename O::V;
@@ -32,7 +31,7 @@ namespace llamql
         const u32x4 *w[RT];
 #pragma unroll
         for (int t = 0; t < RT; ++t)
-            w[t] = weight_tile(static_cast<const bf16 *>(p.w) + (size_t)z * p.w_stride, (size_t)blockIdx.x * RT + t, ksteps, lane);
+            w[t] = weight_tile(static_cast<const bf16 *>(p.w) + (size_t)z * p.w_stride - (t && (block * RT + t) * 16 >= p.N ? (size_t)ksteps * 512 : 0), (size_t)block * RT + t, ksteps, lane);
         u32x4 next[RT][U];
         auto fetch = [&](int s0) __attribute__((always_inline)) {
 #pragma unroll
@@ -68,7 +67,7 @@ namespace llamql
                     const f32x4 v = x[i] * inv * reinterpret_cast<const f32x4 *>(p.norm)[i];
                     const t4 o = __builtin_convertvector(v, t4);
                     *reinterpret_cast<t4 *>(h + (size_t)m * ldh + 4 * i) = o;
-                    if (p.h_out && blockIdx.x == 0)
+                    if (p.h_out && block == 0)
                         *reinterpret_cast<t4 *>(static_cast<T *>(p.h_out) + (size_t)m * p.K + 4 * i) = o;
                 }
             }
@@ -122,11 +121,33 @@ namespace llamql
             }
             const size_t elem = p.out == LLAM_SEQ_OUT_F32 || p.out == LLAM_SEQ_OUT_ADD ? 4 : sizeof(T);
             char *y = static_cast<char *>(p.y) + (size_t)z * p.y_stride * elem;
-            if (RT == 2)
-                store4<T>(p, y, n, blockIdx.x * 16 + 4 * g, gated4(sum[0], sum[RT - 1]));
+            if (RT == 2 && is_gated(p.out))
+                store4<T>(p, y, n, block * 16 + 4 * g, gated4(p, sum[0], sum[RT - 1]));
             else
-                store4<T>(p, y, n, blockIdx.x * 16 + 4 * g, sum[0]);
+            {
+                // (the last tile of an odd number of them is a copy)
+#pragma unroll
+                for (int t = 0; t < RT; ++t)
+                    if ((block * RT + t) * 16 < p.N)
+                        store4<T>(p, y, n, (block * RT + t) * 16 + 4 * g, sum[t]);
+            }
         }
+    }
+
+    template <typename T, int NW, int RT, bool NORM>
+    __global__ void __launch_bounds__(NW * 64)
+        linear_small_kernel(LinearArgs p)
+    {
+        linear_small_tile<T, NW, RT, NORM>(p, blockIdx.x);
+    }
+
+    // Two layers over the same rows: the first `blocks` workgroups belong to p.
+    template <typename T, int NW, bool NORM>
+    __global__ void __launch_bounds__(NW * 64)
+        linear_small_pair_kernel(LinearArgs p, LinearArgs second, int blocks)
+    {
+        const bool other = (int)blockIdx.x >= blocks;
+        linear_small_tile<T, NW, 2, NORM>(other ? second : p, other ? (int)blockIdx.x - blocks : (int)blockIdx.x);
     }
 
     namespace
@@ -144,13 +165,33 @@ namespace llamql
         template <typename T>
         bool small_dispatch(const char *fn, const LinearArgs &a, int batch, hipStream_t st)
         {
-            const bool gated = a.out == LLAM_SEQ_OUT_GATED;
+            const bool gated = is_gated(a.out);
             const bool wide = a.K >= 1024;
             if (a.norm)
                 return gated ? small_launch<T, 8, 2, true>(fn, a, batch, st) : small_launch<T, 8, 1, true>(fn, a, batch, st);
             if (gated)
                 return small_launch<T, 8, 2, false>(fn, a, batch, st);
             return wide ? small_launch<T, 8, 1, false>(fn, a, batch, st) : small_launch<T, 4, 1, false>(fn, a, batch, st);
+        }
+    } // namespace
+
+    namespace
+    {
+        template <typename T, bool NORM>
+        bool small_pair_launch(const char *fn, const LinearArgs &a, const LinearArgs &b, hipStream_t st)
+        {
+            static LdsGrant grant;
+            const size_t lds = NORM ? (size_t)a.M * (a.K + 16 / sizeof(T)) * sizeof(T) : 0;
+            if (lds > 32 * 1024 && allow_lds(grant, reinterpret_cast<const void *>(&linear_small_pair_kernel<T, 8, NORM>), 64 * 1024) != hipSuccess)
+                return fail(fn, "cannot reserve %zu bytes of LDS", lds);
+            const int blocks = ceil_div(a.N, 32);
+            hipLaunchKernelGGL((linear_small_pair_kernel<T, 8, NORM>), dim3(blocks + ceil_div(b.N, 32)), dim3(512), lds, st, a, b, blocks);
+            return launched(fn);
+        }
+        template <typename T>
+        bool small_pair_dispatch(const char *fn, const LinearArgs &a, const LinearArgs &b, hipStream_t st)
+        {
+            return a.norm ? small_pair_launch<T, true>(fn, a, b, st) : small_pair_launch<T, false>(fn, a, b, st);
         }
     } // namespace
 
@@ -301,14 +342,14 @@ namespace llamql
             const int m = mt * BM + wm * (BM / 2) + i * 16 + c;
             if (m >= rows)
                 continue;
-            if (p.out == LLAM_SEQ_OUT_GATED)
+            if (is_gated(p.out))
             {
 #pragma unroll
                 for (int j = 0; j < TN; j += 2)
                 {
                     const int tile = nt * (BN / 16) + wn * TN + j;
                     if (tile < w_tiles)
-                        store4<T>(p, y, row0 + m, tile * 8 + 4 * g, gated4(acc[j][i], acc[j + 1][i]));
+                        store4<T>(p, y, row0 + m, tile * 8 + 4 * g, gated4(p, acc[j][i], acc[j + 1][i]));
                 }
             }
             else
@@ -354,36 +395,66 @@ namespace llamql
 
 using namespace llamql;
 
+namespace
+{
+    bool linear_args(const char *fn, const llam_seq_linear_args *a, int dtype, LinearArgs &p)
+    {
+        if (!a || !a->d_a || !a->d_w || !a->d_y)
+            return fail(fn, "null pointer");
+        if (a->M < 0 || a->N < 1 || a->K < 1 || a->batch < 1 || a->batch > 65535)
+            return fail(fn, "bad size (M=%d N=%d K=%d batch=%d)", a->M, a->N, a->K, a->batch);
+        if (dtype != LLAM_SEQ_BF16 && dtype != LLAM_SEQ_F32)
+            return fail(fn, "dtype %d", dtype);
+        const int elem = dtype == LLAM_SEQ_F32 ? 4 : 2;
+        const bool gated = is_gated(a->out);
+        if ((a->N % (gated ? 32 : 16)) != 0 || (a->K % PAD) != 0)
+            return fail(fn, "N=%d must be a multiple of %d and K=%d of %d", a->N, gated ? 32 : 16, a->K, PAD);
+        if (a->out < LLAM_SEQ_OUT_F32 || a->out > LLAM_SEQ_OUT_GATED_CLAMP)
+            return fail(fn, "output kind %d", a->out);
+        if (a->lda < a->K || a->ldy < (gated ? a->N / 2 : a->N))
+            return fail(fn, "row strides smaller than the rows");
+        if (!aligned16(a->d_a) || !aligned16(a->d_w) || !aligned16(a->d_y) || ((a->lda * (a->d_norm ? 4 : elem)) % 16) != 0 ||
+            (a->ldy % 4) != 0 || ((a->a_stride * elem) % 16) != 0 || ((a->w_stride * 2) % 16) != 0 || (a->y_stride % 4) != 0)
+            return fail(fn, "misaligned rows");
+        if (a->d_norm && (a->M > SMALL_M || a->batch != 1 || (long)a->M * a->K > NORM_FUSE_MAX || a->k_real < 1 || !aligned16(a->d_norm)))
+            return fail(fn, "a fused norm takes up to %d rows and %d values, unbatched", SMALL_M, NORM_FUSE_MAX);
+        p = LinearArgs{};
+        p.a = a->d_a, p.w = a->d_w, p.y = a->d_y, p.bias = a->d_bias, p.norm = a->d_norm, p.h_out = a->d_h_out;
+        p.eps = a->eps, p.k_real = a->k_real, p.M = a->M, p.N = a->N, p.K = a->K, p.lda = a->lda, p.ldy = a->ldy;
+        p.out = a->out, p.limit = a->limit, p.a_stride = a->a_stride, p.w_stride = a->w_stride, p.y_stride = a->y_stride;
+        p.source_div = 1;
+        return true;
+    }
+} // namespace
+
 extern "C" bool llam_seq_linear(const llam_seq_linear_args *a, int dtype, int device_id, void *stream)
 {
     static const char *fn = "llam_seq_linear";
-    if (!a || !a->d_a || !a->d_w || !a->d_y)
-        return fail(fn, "null pointer");
-    if (a->M < 0 || a->N < 1 || a->K < 1 || a->batch < 1 || a->batch > 65535)
-        return fail(fn, "bad size (M=%d N=%d K=%d batch=%d)", a->M, a->N, a->K, a->batch);
+    LinearArgs p;
+    if (!linear_args(fn, a, dtype, p))
+        return false;
     if (a->M == 0)
         return true;
-    if (dtype != LLAM_SEQ_BF16 && dtype != LLAM_SEQ_F32)
-        return fail(fn, "dtype %d", dtype);
-    const int elem = dtype == LLAM_SEQ_F32 ? 4 : 2;
-    const bool gated = a->out == LLAM_SEQ_OUT_GATED;
-    if ((a->N % (gated ? 32 : 16)) != 0 || (a->K % PAD) != 0)
-        return fail(fn, "N=%d must be a multiple of %d and K=%d of %d", a->N, gated ? 32 : 16, a->K, PAD);
-    if (a->out < LLAM_SEQ_OUT_F32 || a->out > LLAM_SEQ_OUT_RELU2)
-        return fail(fn, "output kind %d", a->out);
-    if (a->lda < a->K || a->ldy < (gated ? a->N / 2 : a->N))
-        return fail(fn, "row strides smaller than the rows");
-    if (!aligned16(a->d_a) || !aligned16(a->d_w) || !aligned16(a->d_y) || ((a->lda * (a->d_norm ? 4 : elem)) % 16) != 0 ||
-        (a->ldy % 4) != 0 || ((a->a_stride * elem) % 16) != 0 || ((a->w_stride * 2) % 16) != 0 || (a->y_stride % 4) != 0)
-        return fail(fn, "misaligned rows");
-    if (a->d_norm && (a->M > SMALL_M || a->batch != 1 || (long)a->M * a->K > NORM_FUSE_MAX || a->k_real < 1 || !aligned16(a->d_norm)))
-        return fail(fn, "a fused norm takes up to %d rows and %d values, unbatched", SMALL_M, NORM_FUSE_MAX);
     if (!set_device(fn, device_id))
         return false;
-    LinearArgs p{};
-    p.a = a->d_a, p.w = a->d_w, p.y = a->d_y, p.bias = a->d_bias, p.norm = a->d_norm, p.h_out = a->d_h_out;
-    p.eps = a->eps, p.k_real = a->k_real, p.M = a->M, p.N = a->N, p.K = a->K, p.lda = a->lda, p.ldy = a->ldy;
-    p.out = a->out, p.a_stride = a->a_stride, p.w_stride = a->w_stride, p.y_stride = a->y_stride, p.source_div = 1;
     return a->M <= SMALL_M ? linear_small(fn, p, a->batch, dtype, as_stream(stream))
                            : linear_tiled(fn, p, a->batch, dtype, as_stream(stream));
+}
+
+extern "C" bool llam_seq_linear_pair(const llam_seq_linear_args *a, const llam_seq_linear_args *b, int dtype, int device_id, void *stream)
+{
+    static const char *fn = "llam_seq_linear_pair";
+    LinearArgs p, q;
+    if (!linear_args(fn, a, dtype, p) || !linear_args(fn, b, dtype, q))
+        return false;
+    if (p.M != q.M || p.K != q.K || a->batch != 1 || b->batch != 1 || !p.norm != !q.norm)
+        return fail(fn, "the layers of a pair have the same rows and columns (M=%d, %d K=%d, %d)", p.M, q.M, p.K, q.K);
+    if (p.M == 0)
+        return true;
+    if (!set_device(fn, device_id))
+        return false;
+    hipStream_t st = as_stream(stream);
+    if (p.M <= SMALL_M)
+        return dtype == LLAM_SEQ_F32 ? small_pair_dispatch<float>(fn, p, q, st) : small_pair_dispatch<bf16>(fn, p, q, st);
+    return linear_tiled(fn, p, 1, dtype, st) && linear_tiled(fn, q, 1, dtype, st);
 }

@@ -29,6 +29,7 @@ namespace llamql
         const float *gate_bias, *norm;
         float *state, *m;
         void *y;
+        int ldy;
         int heads, dim, vdim, vdim_real;
         float q_scale, gate_cap, eps;
         const int32_t *row0, *ntok, *slot, *pos;
@@ -566,7 +567,7 @@ namespace llamql
         const float scale = 1.0f / sqrtf(sum / (float)p.vdim_real + p.eps);
         const float *gate = row + (size_t)p.heads * (2 * p.dim + p.vdim) + h * p.vdim;
         typedef T t4 __attribute__((ext_vector_type(4)));
-        T *y = static_cast<T *>(p.y) + ((size_t)r * p.heads + h) * p.vdim;
+        T *y = static_cast<T *>(p.y) + (size_t)r * p.ldy + h * p.vdim;
         for (int d = d0; d < p.vdim; d += 512)
         {
             f32x4 o = (d == d0 ? kept : total(d) * inv) * scale * *reinterpret_cast<const f32x4 *>(p.norm + h * p.vdim + d);
@@ -621,11 +622,13 @@ namespace llamql
                 return fail(fn, "heads=%d dim=%d vdim=%d: dim up to 512, both multiples of %d", a->heads, a->dim, a->vdim, PAD);
             if (a->ldp < a->heads * (2 * a->dim + 2 * a->vdim + 2) || (a->ldp % 4) != 0 || !aligned16(a->d_proj))
                 return fail(fn, "ldp=%d too small or rows misaligned", a->ldp);
+            if (a->ldy < a->heads * a->vdim || (a->ldy % 8) != 0)
+                return fail(fn, "ldy=%d too small or rows misaligned", a->ldy);
             if (!(a->gate_cap > 0.0f))
                 return fail(fn, "gate_cap must be positive");
             p = MemoryArgs{};
             p.proj = a->d_proj, p.ldp = a->ldp, p.gate_bias = a->d_gate_bias, p.norm = a->d_norm, p.state = a->d_state;
-            p.m = a->d_m, p.y = a->d_y, p.heads = a->heads, p.dim = a->dim, p.vdim = a->vdim, p.vdim_real = a->vdim_real;
+            p.m = a->d_m, p.y = a->d_y, p.ldy = a->ldy, p.heads = a->heads, p.dim = a->dim, p.vdim = a->vdim, p.vdim_real = a->vdim_real;
             p.q_scale = a->q_scale, p.gate_cap = a->gate_cap, p.eps = a->eps;
             p.row0 = e->d_row0, p.ntok = e->d_ntok, p.slot = e->d_slot, p.pos = e->d_pos;
             return true;

@@ -7,19 +7,44 @@ namespace llamql
     constexpr int ROW_THREADS = 256;
 
     __global__ void __launch_bounds__(ROW_THREADS)
-        seq_embed_kernel(const bf16 *__restrict__ table, int vocab, int width, const int32_t *__restrict__ ids,
-                         float *__restrict__ x, int ldx)
+        seq_embed_kernel(llam_seq_embed_args p, const int32_t *__restrict__ ids, float *__restrict__ x, int ldx)
     {
         const int m = blockIdx.y, id = ids[m], c = blockIdx.x * ROW_THREADS + threadIdx.x;
-        const bool ok = id >= 0 && id < vocab;
+        const bool ok = id >= 0 && id < p.vocab;
+        const bf16 *table = static_cast<const bf16 *>(p.d_table), *pairs = static_cast<const bf16 *>(p.d_pairs);
+        long pair = -1;
+        if (pairs)
+        {
+            const int slot = p.d_row_slot[m], pos = p.d_row_pos[m];
+            int32_t *history = p.d_history + (size_t)slot * p.cap;
+            if (pos == 0)
+                pair = p.buckets;
+            else if (pos > 0 && pos < p.cap)
+            {
+                const int before = m > 0 && p.d_row_slot[m - 1] == slot ? ids[m - 1] : history[pos - 1];
+                pair = ((long)before * p.mul_prev + (long)id * p.mul_cur) % p.buckets;
+            }
+            if (blockIdx.x == 0 && threadIdx.x == 0 && pos >= 0 && pos < p.cap)
+                history[pos] = id;
+        }
         if (c < ldx)
-            x[(size_t)m * ldx + c] = ok && c < width ? (float)table[(size_t)id * width + c] : 0.0f;
+        {
+            float v = 0.0f;
+            if (ok && c < p.width)
+            {
+                v = (float)table[(size_t)id * p.width + c] * p.scale;
+                if (pair >= 0)
+                    v += (float)pairs[(size_t)pair * p.width + c];
+            }
+            x[(size_t)m * ldx + c] = v;
+        }
     }
 
     template <typename T>
     __global__ void __launch_bounds__(ROW_THREADS)
         seq_rmsnorm_kernel(const float *__restrict__ x, int ldx, const int32_t *__restrict__ rows,
-                           const float *__restrict__ norm, float eps, int k_real, T *__restrict__ y, int K)
+                           const float *__restrict__ norm, float eps, int k_real, T *__restrict__ y, int K,
+                           const float *__restrict__ norm2, T *__restrict__ y2)
     {
         typedef T t4 __attribute__((ext_vector_type(4)));
         __shared__ float s_sum[ROW_THREADS / 64];
@@ -34,8 +59,14 @@ namespace llamql
         sum = block_sum<ROW_THREADS>(sum, s_sum);
         const float inv = 1.0f / sqrtf(sum / (float)k_real + eps);
         for (int i = threadIdx.x; i < K / 4; i += ROW_THREADS)
+        {
+            const f32x4 v = row[i] * inv;
             *reinterpret_cast<t4 *>(y + (size_t)m * K + 4 * i) =
-                __builtin_convertvector(row[i] * inv * reinterpret_cast<const f32x4 *>(norm)[i], t4);
+                __builtin_convertvector(v * reinterpret_cast<const f32x4 *>(norm)[i], t4);
+            if (norm2)
+                *reinterpret_cast<t4 *>(y2 + (size_t)m * K + 4 * i) =
+                    __builtin_convertvector(v * reinterpret_cast<const f32x4 *>(norm2)[i], t4);
+        }
     }
 
     __global__ void __launch_bounds__(64)
@@ -407,46 +438,62 @@ namespace llamql
 
 using namespace llamql;
 
-extern "C" bool llam_seq_embed(const void *d_table, int vocab, int width, const int32_t *d_ids, float *d_x, int M,
-                               int ldx, int device_id, void *stream)
+extern "C" bool llam_seq_embed(const llam_seq_embed_args *a, const int32_t *d_ids, float *d_x, int M, int ldx, int device_id,
+                               void *stream)
 {
     static const char *fn = "llam_seq_embed";
-    if (M < 0 || vocab < 1 || width < 1 || ldx < width)
-        return fail(fn, "bad size (M=%d vocab=%d width=%d ldx=%d)", M, vocab, width, ldx);
+    if (!a || !a->d_table || !d_ids || !d_x)
+        return fail(fn, "null pointer");
+    if (M < 0 || M > 65535 || a->vocab < 1 || a->width < 1 || ldx < a->width)
+        return fail(fn, "bad size (M=%d vocab=%d width=%d ldx=%d)", M, a->vocab, a->width, ldx);
+    if (a->d_pairs && (!a->d_row_slot || !a->d_row_pos || !a->d_history || a->buckets < 1 || a->cap < 1))
+        return fail(fn, "pairs of tokens need rows, a history and buckets=%d cap=%d of at least 1", a->buckets, a->cap);
     if (M == 0)
         return true;
-    if (!d_table || !d_ids || !d_x)
-        return fail(fn, "null pointer");
     if (!set_device(fn, device_id))
         return false;
-    if (M > 65535)
-        return fail(fn, "M=%d rows", M);
-    hipLaunchKernelGGL(seq_embed_kernel, dim3(ceil_div(ldx, ROW_THREADS), M), dim3(ROW_THREADS), 0, as_stream(stream),
-                       static_cast<const bf16 *>(d_table), vocab, width, d_ids, d_x, ldx);
+    hipLaunchKernelGGL(seq_embed_kernel, dim3(ceil_div(ldx, ROW_THREADS), M), dim3(ROW_THREADS), 0, as_stream(stream), *a, d_ids, d_x, ldx);
     return launched(fn);
 }
+
+namespace
+{
+    bool rmsnorm(const char *fn, const float *d_x, int ldx, const int32_t *d_rows, const float *d_norm, const float *d_norm2, float eps,
+                 int k_real, void *d_y, void *d_y2, int M, int K, int dtype, int device_id, void *stream)
+    {
+        if (M < 0 || K < 1 || k_real < 1 || k_real > K || ldx < K)
+            return fail(fn, "bad size (M=%d K=%d k_real=%d ldx=%d)", M, K, k_real, ldx);
+        if (M == 0)
+            return true;
+        if (!d_x || !d_norm || !d_y)
+            return fail(fn, "null pointer");
+        if ((K % 8) != 0 || (ldx % 4) != 0 || !aligned16(d_x) || !aligned16(d_norm) || !aligned16(d_y) || !aligned16(d_norm2) || !aligned16(d_y2))
+            return fail(fn, "misaligned rows");
+        if (!set_device(fn, device_id))
+            return false;
+        if (dtype == LLAM_SEQ_F32)
+            hipLaunchKernelGGL(seq_rmsnorm_kernel<float>, dim3(M), dim3(ROW_THREADS), 0, as_stream(stream), d_x, ldx, d_rows,
+                               d_norm, eps, k_real, static_cast<float *>(d_y), K, d_norm2, static_cast<float *>(d_y2));
+        else
+            hipLaunchKernelGGL(seq_rmsnorm_kernel<bf16>, dim3(M), dim3(ROW_THREADS), 0, as_stream(stream), d_x, ldx, d_rows,
+                               d_norm, eps, k_real, static_cast<bf16 *>(d_y), K, d_norm2, static_cast<bf16 *>(d_y2));
+        return launched(fn);
+    }
+} // namespace
 
 extern "C" bool llam_seq_rmsnorm(const float *d_x, int ldx, const int32_t *d_rows, const float *d_norm, float eps,
                                  int k_real, void *d_y, int M, int K, int dtype, int device_id, void *stream)
 {
-    static const char *fn = "llam_seq_rmsnorm";
-    if (M < 0 || K < 1 || k_real < 1 || k_real > K || ldx < K)
-        return fail(fn, "bad size (M=%d K=%d k_real=%d ldx=%d)", M, K, k_real, ldx);
-    if (M == 0)
-        return true;
-    if (!d_x || !d_norm || !d_y)
+    return rmsnorm("llam_seq_rmsnorm", d_x, ldx, d_rows, d_norm, nullptr, eps, k_real, d_y, nullptr, M, K, dtype, device_id, stream);
+}
+
+extern "C" bool llam_seq_rmsnorm_pair(const float *d_x, int ldx, const float *d_norm_a, const float *d_norm_b, float eps, int k_real,
+                                      void *d_ya, void *d_yb, int M, int K, int dtype, int device_id, void *stream)
+{
+    static const char *fn = "llam_seq_rmsnorm_pair";
+    if (!d_norm_b || !d_yb)
         return fail(fn, "null pointer");
-    if ((K % 8) != 0 || (ldx % 4) != 0 || !aligned16(d_x) || !aligned16(d_norm) || !aligned16(d_y))
-        return fail(fn, "misaligned rows");
-    if (!set_device(fn, device_id))
-        return false;
-    if (dtype == LLAM_SEQ_F32)
-        hipLaunchKernelGGL(seq_rmsnorm_kernel<float>, dim3(M), dim3(ROW_THREADS), 0, as_stream(stream), d_x, ldx, d_rows,
-                           d_norm, eps, k_real, static_cast<float *>(d_y), K);
-    else
-        hipLaunchKernelGGL(seq_rmsnorm_kernel<bf16>, dim3(M), dim3(ROW_THREADS), 0, as_stream(stream), d_x, ldx, d_rows,
-                           d_norm, eps, k_real, static_cast<bf16 *>(d_y), K);
-    return launched(fn);
+    return rmsnorm(fn, d_x, ldx, nullptr, d_norm_a, d_norm_b, eps, k_real, d_ya, d_yb, M, K, dtype, device_id, stream);
 }
 
 extern "C" size_t llam_seq_experts_scratch_bytes(int max_rows, int experts, int top, int ff, int shared_ff, int N)

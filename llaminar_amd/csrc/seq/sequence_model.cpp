@@ -47,6 +47,11 @@ namespace
 
     int pad(int n, int to) { return (n + to - 1) / to * to; }
     int P(int n) { return pad(n, 64); }
+    int A(int n) { return n <= 64 ? 64 : n <= 128 ? 128 : 256; } // heads of the grouped-query attention
+    bool gated(int ffn) { return ffn == LLAM_FFN_GATED || ffn == LLAM_FFN_GATED_CLAMP; }
+    int value_pad(const llam_seqm_layer &w) { return w.mixer == LLAM_MIXER_ATTENTION ? A(w.vdim) : P(w.vdim); }
+    // columns of the buffer a mixer writes its heads to: a parallel layer's feed-forward lies behind them
+    int mix_columns(const llam_seqm_layer &w) { return w.heads * value_pad(w) + (w.parallel && w.ffn ? P(w.ff) : 0); }
 
     constexpr int ROW_MAX = 16;         // rows of the row-at-a-time kernels
     constexpr int NORM_FUSE_MAX = 8192; // values a linear layer norms by itself
@@ -64,13 +69,16 @@ namespace
         std::vector<void *> owned;
         size_t owned_bytes = 0;
         std::vector<void *> cache;   // per layer: latent cache (its own), else null
-        std::vector<float *> memory; // per layer: matrix memory
-        std::vector<float *> mem_m;
+        std::vector<void *> values;  // per attention layer: the cache's values (keys in `cache`)
+        std::vector<int> cache_rows; // per attention layer: rows of its ring
+        std::vector<float *> memory; // per layer: matrix memory, or state of the delta rule
+        std::vector<float *> mem_m;  // per layer: running maxima, or recent inputs of the convolution
+        int32_t *history = nullptr;  // ids of every slot, where pairs of them are embedded
         size_t slot_bytes = 0;
 
         int wp = 0, vp = 0, elem = 2;
         float *x = nullptr, *in = nullptr, *z = nullptr, *logits = nullptr, *lat_scratch = nullptr;
-        void *h = nullptr, *q = nullptr, *qlat = nullptr, *olat = nullptr, *mix = nullptr, *act = nullptr;
+        void *h = nullptr, *h2 = nullptr, *q = nullptr, *qlat = nullptr, *olat = nullptr, *mix = nullptr, *act = nullptr;
         void *scratch = nullptr, *arg_scratch = nullptr;
         size_t lat_floats = 0, scratch_bytes = 0;
         // integers of a step: ids, slot and position per row; first row, tokens, slot, position per entry; wanted rows
@@ -146,9 +154,10 @@ namespace
 
         bool linear(const void *a, int lda, const void *w, int N, int K, void *y, int ldy, int out, int M,
                     const float *bias = nullptr, const float *norm = nullptr, int k_real = 0, void *h_out = nullptr,
-                    int batch = 1, long as = 0, long ws = 0, long ys = 0)
+                    int batch = 1, long as = 0, long ws = 0, long ys = 0, float limit = 0.0f)
         {
             llam_seq_linear_args l{};
+            l.limit = limit;
             l.d_a = a, l.lda = lda, l.d_w = w, l.N = N, l.K = K, l.d_y = y, l.ldy = ldy, l.out = out, l.M = M;
             l.d_bias = bias, l.d_norm = norm, l.k_real = k_real, l.eps = c.eps, l.d_h_out = h_out;
             l.batch = batch, l.a_stride = as, l.w_stride = ws, l.y_stride = ys;
@@ -159,13 +168,83 @@ namespace
 
         // y = W rms(x) norm: in one launch for a few rows
         bool norm_linear(const float *x, int ldx, const float *norm, int k_real, const void *w, int N, void *y, int ldy,
-                         int out, int M, const float *bias = nullptr, bool keep_h = false)
+                         int out, int M, const float *bias = nullptr, bool keep_h = false, float limit = 0.0f)
         {
             const int K = P(k_real);
             if (fused(M, K))
-                return linear(x, ldx, w, N, K, y, ldy, out, M, bias, norm, k_real, keep_h ? md.h : nullptr);
+                return linear(x, ldx, w, N, K, y, ldy, out, M, bias, norm, k_real, keep_h ? md.h : nullptr, 1, 0, 0, 0, limit);
             return forward(fn, llam_seq_rmsnorm(x, ldx, nullptr, norm, c.eps, k_real, md.h, M, K, c.dtype, c.device_id, st)) &&
-                   linear(md.h, K, w, N, K, y, ldy, out, M, bias);
+                   linear(md.h, K, w, N, K, y, ldy, out, M, bias, nullptr, 0, nullptr, 1, 0, 0, 0, limit);
+        }
+
+        int gated_out(const llam_seqm_layer &w) { return w.ffn == LLAM_FFN_GATED_CLAMP ? LLAM_SEQ_OUT_GATED_CLAMP : LLAM_SEQ_OUT_GATED; }
+
+        // the mixer's projections of x; a parallel layer's gate and up projections go with them
+        bool project(const llam_seqm_layer &w, int n_in, const Step &s)
+        {
+            if (!w.parallel || w.ffn == LLAM_FFN_NONE)
+                return norm_linear(md.x, md.wp, w.norm1, c.width, w.w_in, n_in, md.in, n_in, LLAM_SEQ_OUT_F32, s.M);
+            const int K = md.wp, fp = P(w.ff), ldm = mix_columns(w);
+            llam_seq_linear_args a{}, f{};
+            const bool fuse = fused(s.M, K);
+            if (!fuse && !forward(fn, llam_seq_rmsnorm_pair(md.x, md.wp, w.norm1, w.norm2, c.eps, c.width, md.h, md.h2, s.M, K, c.dtype, c.device_id, st)))
+                return false;
+            a.d_a = fuse ? md.x : md.h, a.d_w = w.w_in, a.d_y = md.in, a.N = n_in, a.ldy = n_in, a.out = LLAM_SEQ_OUT_F32;
+            f.d_a = fuse ? md.x : md.h2, f.d_w = w.w_up, f.N = 2 * fp, f.ldy = ldm, f.out = gated_out(w), f.limit = w.limit;
+            f.d_y = static_cast<char *>(md.mix) + (size_t)(ldm - fp) * md.elem;
+            a.d_norm = fuse ? w.norm1 : nullptr, f.d_norm = fuse ? w.norm2 : nullptr;
+            for (llam_seq_linear_args *l : {&a, &f})
+                l->M = s.M, l->K = K, l->lda = fuse ? md.wp : K, l->k_real = c.width, l->eps = c.eps, l->batch = 1;
+            return forward(fn, llam_seq_linear_pair(&a, &f, c.dtype, c.device_id, st));
+        }
+
+        // x += W_out of the mixer's heads (and of a parallel layer's feed-forward)
+        bool add_output(const llam_seqm_layer &w, const Step &s)
+        {
+            const int K = mix_columns(w);
+            return linear(md.mix, K, w.w_out, md.wp, K, md.x, md.wp, LLAM_SEQ_OUT_ADD, s.M);
+        }
+
+        bool attention(const llam_seqm_layer &w, int index, const Step &s)
+        {
+            const bool own = w.kv_from < 0;
+            const int from = own ? index : w.kv_from;
+            llam_seq_attention_args a{};
+            a.heads = w.heads, a.kv_heads = w.kv_heads, a.dim = A(w.dim), a.vdim = A(w.vdim);
+            a.ring = md.cache_rows[from], a.chunk = w.chunk, a.scale = w.scale, a.d_k = md.cache[from], a.d_v = md.values[from];
+            const int n_in = w.heads * a.dim + (own ? w.kv_heads * (a.dim + a.vdim) : 0), ldm = mix_columns(w);
+            if (!project(w, n_in, s) ||
+                !forward(fn, llam_seq_rotary(&a, md.in, n_in, own, w.turns, w.rot_dims, s.row_slot, s.row_pos, md.q, s.M, c.dtype, c.device_id, st)))
+                return false;
+            const llam_seq_entries e = md.entries();
+            if (s.single && !forward(fn, llam_seq_attention(&a, md.q, &e, 0, s.single, 1, s.max_len, md.mix, ldm, md.lat_scratch, md.lat_floats,
+                                                            c.dtype, c.device_id, st)))
+                return false;
+            for (size_t k = 0; k < s.portions.size(); ++k)
+                if (!forward(fn, llam_seq_attention(&a, md.q, &e, s.single + (int)k, 1, s.portions[k].first, s.portions[k].second, md.mix, ldm,
+                                                    md.lat_scratch, md.lat_floats, c.dtype, c.device_id, st)))
+                    return false;
+            return add_output(w, s);
+        }
+
+        bool delta(const llam_seqm_layer &w, int index, const Step &s)
+        {
+            const int H = w.heads, G = w.kv_heads, dp = P(w.dim), vp = P(w.vdim);
+            const int n_in = pad(2 * G * dp + 2 * H * vp + 2 * H, 16);
+            if (!project(w, n_in, s))
+                return false;
+            llam_seq_delta_args a{};
+            a.d_proj = md.in, a.ldp = n_in, a.d_conv = w.conv, a.d_a_log = w.a_log, a.d_dt_bias = w.dt_bias, a.d_norm = w.head_norm;
+            a.d_state = md.memory[index], a.d_recent = md.mem_m[index], a.d_y = md.mix, a.ldy = mix_columns(w);
+            a.heads = H, a.kv_heads = G, a.dim = dp, a.vdim = vp, a.dim_real = w.dim, a.vdim_real = w.vdim, a.taps = w.taps, a.eps = c.eps;
+            const llam_seq_entries e = md.entries();
+            if (s.single && !forward(fn, llam_seq_delta_decode(&a, &e, 0, s.single, c.dtype, c.device_id, st)))
+                return false;
+            for (size_t k = 0; k < s.portions.size(); ++k)
+                if (!forward(fn, llam_seq_delta_prefill(&a, &e, s.single + (int)k, s.portions[k].first, md.scratch, md.scratch_bytes, c.dtype,
+                                                        c.device_id, st)))
+                    return false;
+            return add_output(w, s);
         }
 
         bool latent(const llam_seqm_layer &w, int index, const Step &s)
@@ -173,7 +252,7 @@ namespace
             const int H = w.heads, dp = P(w.dim), vp = P(w.vdim), qp = P(w.q_rank), rp = P(w.kv_rank);
             const bool own = w.kv_from < 0;
             const int n_in = qp + (own ? rp : 0);
-            if (!norm_linear(md.x, md.wp, w.norm1, c.width, w.w_in, n_in, md.in, n_in, LLAM_SEQ_OUT_F32, s.M))
+            if (!project(w, n_in, s))
                 return false;
             void *cache = md.cache[own ? index : w.kv_from];
             if (own && !forward(fn, llam_seq_latent_append(md.in + qp, n_in, w.kv_norm, c.eps, w.kv_rank, s.row_slot, s.row_pos,
@@ -192,20 +271,20 @@ namespace
                                                            s.portions[k].second, H, rp, c.cap, w.scale, md.olat, md.lat_scratch,
                                                            md.lat_floats, c.dtype, c.device_id, st)))
                     return false;
-            return linear(md.olat, H * rp, w.w_uv, vp, rp, md.mix, H * vp, LLAM_SEQ_OUT_ELEM, s.M, nullptr, nullptr, 0, nullptr, H,
+            return linear(md.olat, H * rp, w.w_uv, vp, rp, md.mix, mix_columns(w), LLAM_SEQ_OUT_ELEM, s.M, nullptr, nullptr, 0, nullptr, H,
                           rp, (long)vp * rp, vp) &&
-                   linear(md.mix, H * vp, w.w_out, md.wp, H * vp, md.x, md.wp, LLAM_SEQ_OUT_ADD, s.M);
+                   add_output(w, s);
         }
 
         bool memory(const llam_seqm_layer &w, int index, const Step &s)
         {
             const int H = w.heads, dp = P(w.dim), vp = P(w.vdim);
             const int n_in = pad(2 * H * (dp + vp) + 2 * H, 16);
-            if (!norm_linear(md.x, md.wp, w.norm1, c.width, w.w_in, n_in, md.in, n_in, LLAM_SEQ_OUT_F32, s.M))
+            if (!project(w, n_in, s))
                 return false;
             llam_seq_memory_args a{};
             a.d_proj = md.in, a.ldp = n_in, a.d_gate_bias = w.gate_bias, a.d_norm = w.head_norm;
-            a.d_state = md.memory[index], a.d_m = md.mem_m[index], a.d_y = md.mix;
+            a.d_state = md.memory[index], a.d_m = md.mem_m[index], a.d_y = md.mix, a.ldy = mix_columns(w);
             a.heads = H, a.dim = dp, a.vdim = vp, a.vdim_real = w.vdim;
             a.q_scale = w.scale, a.gate_cap = w.gate_cap, a.eps = c.eps;
             const llam_seq_entries e = md.entries();
@@ -215,14 +294,14 @@ namespace
                 if (!forward(fn, llam_seq_memory_prefill(&a, &e, s.single + (int)k, s.portions[k].first, md.scratch, md.scratch_bytes,
                                                          c.dtype, c.device_id, st)))
                     return false;
-            return linear(md.mix, H * vp, w.w_out, md.wp, H * vp, md.x, md.wp, LLAM_SEQ_OUT_ADD, s.M);
+            return add_output(w, s);
         }
 
         bool ffn(const llam_seqm_layer &w, const Step &s)
         {
             const int fp = P(w.ff), wp = md.wp;
-            if (w.ffn == LLAM_FFN_GATED)
-                return norm_linear(md.x, wp, w.norm2, c.width, w.w_up, 2 * fp, md.act, fp, LLAM_SEQ_OUT_GATED, s.M) &&
+            if (gated(w.ffn))
+                return norm_linear(md.x, wp, w.norm2, c.width, w.w_up, 2 * fp, md.act, fp, gated_out(w), s.M, nullptr, false, w.limit) &&
                        linear(md.act, fp, w.w_down, wp, fp, md.x, wp, LLAM_SEQ_OUT_ADD, s.M);
             const int zp = pad(w.experts + (w.shared_ff ? 1 : 0), 16), sp = w.shared_ff ? P(w.shared_ff) : 0;
             if (!norm_linear(md.x, wp, w.norm2, c.width, w.w_router, zp, md.z, zp, LLAM_SEQ_OUT_F32, s.M, w.router_bias, true))
@@ -238,14 +317,20 @@ namespace
 
         bool layers(const Step &s)
         {
-            if (!forward(fn, llam_seq_embed(md.globals.embed, c.vocab, c.width, md.ids(), md.x, s.M, md.wp, c.device_id, st)))
+            const llam_seqm_globals &gl = md.globals;
+            llam_seq_embed_args em{};
+            em.d_table = gl.embed, em.vocab = c.vocab, em.width = c.width, em.scale = gl.embed_scale;
+            em.d_pairs = gl.pairs, em.buckets = gl.buckets, em.mul_prev = gl.mul_prev, em.mul_cur = gl.mul_cur;
+            em.d_row_slot = s.row_slot, em.d_row_pos = s.row_pos, em.d_history = md.history, em.cap = c.cap;
+            if (!forward(fn, llam_seq_embed(&em, md.ids(), md.x, s.M, md.wp, c.device_id, st)))
                 return false;
             for (int l = 0; l < c.n_layers; ++l)
             {
                 const llam_seqm_layer &w = md.layers[l];
-                if (!(w.mixer == LLAM_MIXER_LATENT_ATTENTION ? latent(w, l, s) : memory(w, l, s)))
+                if (!(w.mixer == LLAM_MIXER_LATENT_ATTENTION ? latent(w, l, s) : w.mixer == LLAM_MIXER_MATRIX_MEMORY ? memory(w, l, s)
+                      : w.mixer == LLAM_MIXER_ATTENTION ? attention(w, l, s) : delta(w, l, s)))
                     return false;
-                if (w.ffn != LLAM_FFN_NONE && !ffn(w, s))
+                if (w.ffn != LLAM_FFN_NONE && !w.parallel && !ffn(w, s))
                     return false;
                 if (md.trace && !hip_ok(fn, "hipMemcpy2DAsync", hipMemcpy2DAsync(md.trace + (size_t)l * s.M * c.width, (size_t)c.width * 4, md.x,
                                                                                  (size_t)md.wp * 4, (size_t)c.width * 4, s.M,
@@ -374,13 +459,37 @@ extern "C" bool llam_seqm_set_layer(void *model, int layer, const llam_seqm_laye
         if (!w->gate_bias || !w->head_norm || !(w->gate_cap > 0.0f) || P(w->dim) > 512)
             return fail(fn, "layer %d: tensors of the matrix memory are missing, or dim=%d above 512", layer, w->dim);
     }
+    else if (w->mixer == LLAM_MIXER_ATTENTION)
+    {
+        if (w->kv_heads < 1 || (w->heads % w->kv_heads) != 0 || w->dim > 256 || w->vdim > 256)
+            return fail(fn, "layer %d: heads=%d must be a multiple of kv_heads=%d, dim=%d and vdim=%d at most 256", layer, w->heads, w->kv_heads, w->dim, w->vdim);
+        if (w->rot_dims < 0 || (w->rot_dims % 2) != 0 || w->rot_dims > w->dim || (w->rot_dims && !w->turns) || w->chunk < 0)
+            return fail(fn, "layer %d: rot_dims=%d chunk=%d", layer, w->rot_dims, w->chunk);
+        if (w->kv_from >= 0)
+        {
+            if (w->kv_from >= layer || !md->layer_set[w->kv_from])
+                return fail(fn, "layer %d: kv_from %d is not an earlier layer", layer, w->kv_from);
+            const llam_seqm_layer &from = md->layers[w->kv_from];
+            if (from.mixer != LLAM_MIXER_ATTENTION || from.kv_from >= 0 || from.kv_heads != w->kv_heads || from.dim != w->dim || from.vdim != w->vdim)
+                return fail(fn, "layer %d: layer %d has no keys and values of its own of these sizes", layer, w->kv_from);
+        }
+    }
+    else if (w->mixer == LLAM_MIXER_DELTA)
+    {
+        if (w->kv_heads < 1 || (w->heads % w->kv_heads) != 0 || w->dim > 256 || w->vdim > 4096 || w->taps < 1 || w->taps > 1024)
+            return fail(fn, "layer %d: heads=%d must be a multiple of kv_heads=%d, dim=%d at most 256, vdim=%d at most 4096, taps=%d", layer, w->heads, w->kv_heads, w->dim, w->vdim, w->taps);
+        if (!w->conv || !w->a_log || !w->dt_bias || !w->head_norm)
+            return fail(fn, "layer %d: tensors of the delta rule are missing", layer);
+    }
     else
         return fail(fn, "layer %d: mixer kind %d", layer, w->mixer);
     if (w->ffn != LLAM_FFN_NONE)
     {
-        if (w->ffn != LLAM_FFN_GATED && w->ffn != LLAM_FFN_EXPERTS)
+        if (!gated(w->ffn) && w->ffn != LLAM_FFN_EXPERTS)
             return fail(fn, "layer %d: feed-forward kind %d", layer, w->ffn);
-        if (w->ff < 1 || !w->norm2 || !w->w_up || !w->w_down)
+        if (w->parallel && !gated(w->ffn))
+            return fail(fn, "layer %d: a parallel layer takes a gated feed-forward", layer);
+        if (w->ff < 1 || !w->norm2 || !w->w_up || (!w->w_down && !w->parallel))
             return fail(fn, "layer %d: sizes or tensors of the feed-forward are missing", layer);
         if (w->ffn == LLAM_FFN_EXPERTS &&
             (w->experts < 1 || w->experts > 1024 || w->top < 1 || w->top > w->experts || w->top > 64 || w->shared_ff < 0 || !w->w_router || !w->router_bias ||
@@ -396,7 +505,7 @@ extern "C" bool llam_seqm_set_globals(void *model, const llam_seqm_globals *g)
 {
     static const char *fn = "set_globals";
     Model *md = static_cast<Model *>(model);
-    if (!md || !g || !g->embed || !g->final_norm || !g->head || md->ready)
+    if (!md || !g || !g->embed || !g->final_norm || !g->head || md->ready || (g->pairs && g->buckets < 1))
         return fail(fn, "bad arguments");
     for (int l = 0; l < md->cfg.n_layers; ++l)
         if (!md->layer_set[l])
@@ -406,11 +515,13 @@ extern "C" bool llam_seqm_set_globals(void *model, const llam_seqm_globals *g)
         return false;
     md->globals = *g;
     const size_t M = c.max_rows, elem = md->elem;
+    bool parallel = false;
     size_t n_in = 0, q = 0, lat = 0, mix = 0, act = 0, z = 16, h = md->wp, latf = 0, scratch = 0;
     for (const llam_seqm_layer &w : md->layers)
     {
         const size_t H = w.heads, dp = P(w.dim), vp = P(w.vdim);
-        mix = std::max(mix, H * vp);
+        mix = std::max(mix, (size_t)mix_columns(w));
+        parallel |= w.parallel && w.ffn;
         if (w.mixer == LLAM_MIXER_LATENT_ATTENTION)
         {
             const size_t rp = P(w.kv_rank);
@@ -420,12 +531,23 @@ extern "C" bool llam_seqm_set_globals(void *model, const llam_seqm_globals *g)
             lat = std::max(lat, H * rp);
             latf = std::max(latf, llam_seq_latent_scratch_floats(c.max_rows, c.slots, w.heads, (int)rp, c.cap));
         }
+        else if (w.mixer == LLAM_MIXER_ATTENTION)
+        {
+            n_in = std::max(n_in, H * A(w.dim) + (w.kv_from < 0 ? (size_t)w.kv_heads * (A(w.dim) + A(w.vdim)) : 0));
+            q = std::max(q, H * A(w.dim));
+            latf = std::max(latf, llam_seq_attention_scratch_floats(A(w.vdim)));
+        }
+        else if (w.mixer == LLAM_MIXER_DELTA)
+        {
+            n_in = std::max(n_in, (size_t)pad((int)(2 * w.kv_heads * dp + 2 * H * vp + 2 * H), 16));
+            scratch = std::max(scratch, llam_seq_delta_scratch_bytes(c.max_rows, w.heads, w.kv_heads, (int)dp, (int)vp));
+        }
         else
         {
             n_in = std::max(n_in, (size_t)pad((int)(2 * H * (dp + vp) + 2 * H), 16));
             scratch = std::max(scratch, llam_seq_memory_scratch_bytes(std::max(c.max_rows, c.slots), w.heads, (int)dp, (int)vp));
         }
-        if (w.ffn == LLAM_FFN_GATED)
+        if (gated(w.ffn) && !w.parallel)
             act = std::max(act, (size_t)P(w.ff));
         if (w.ffn == LLAM_FFN_EXPERTS)
         {
@@ -436,7 +558,7 @@ extern "C" bool llam_seqm_set_globals(void *model, const llam_seqm_globals *g)
     }
     md->lat_floats = latf;
     md->scratch_bytes = scratch;
-    bool ok = (md->x = (float *)md->take(fn, M * md->wp * 4)) && (md->h = md->take(fn, M * h * elem)) &&
+    bool ok = (md->x = (float *)md->take(fn, M * md->wp * 4)) && (md->h = md->take(fn, M * h * elem)) && (md->h2 = md->take(fn, parallel ? M * md->wp * elem : 0)) &&
               (md->in = (float *)md->take(fn, M * n_in * 4)) && (md->q = md->take(fn, M * q * elem)) &&
               (md->qlat = md->take(fn, M * lat * elem)) && (md->olat = md->take(fn, M * lat * elem)) &&
               (md->mix = md->take(fn, M * mix * elem)) && (md->act = md->take(fn, M * act * elem)) &&
@@ -452,6 +574,24 @@ extern "C" bool llam_seqm_set_globals(void *model, const llam_seqm_globals *g)
     md->cache.assign(c.n_layers, nullptr);
     md->memory.assign(c.n_layers, nullptr);
     md->mem_m.assign(c.n_layers, nullptr);
+    md->values.assign(c.n_layers, nullptr);
+    md->cache_rows.assign(c.n_layers, 0);
+    if (g->pairs)
+    {
+        if (!(md->history = (int32_t *)md->take(fn, (size_t)c.slots * c.cap * 4)))
+            return false;
+        md->slot_bytes += (size_t)c.cap * 4;
+    }
+    // rows an attention cache must keep: what the widest mask of its readers shows the first token of a step, and the step
+    for (int l = 0; l < c.n_layers; ++l)
+    {
+        const llam_seqm_layer &w = md->layers[l];
+        if (w.mixer != LLAM_MIXER_ATTENTION)
+            continue;
+        const long sight = w.chunk > 0 ? std::min<long>(c.cap, (long)w.chunk - 1 + c.max_rows) : c.cap;
+        int &ring = md->cache_rows[w.kv_from >= 0 ? w.kv_from : l];
+        ring = std::max(ring, pad((int)sight, 128));
+    }
     for (int l = 0; l < c.n_layers; ++l)
     {
         const llam_seqm_layer &w = md->layers[l];
@@ -463,6 +603,23 @@ extern "C" bool llam_seqm_set_globals(void *model, const llam_seqm_globals *g)
             if (!(md->cache[l] = md->take(fn, per * c.slots)))
                 return false;
             md->slot_bytes += per;
+        }
+        else if (w.mixer == LLAM_MIXER_ATTENTION)
+        {
+            if (w.kv_from >= 0)
+                continue;
+            const size_t rows = (size_t)w.kv_heads * md->cache_rows[l], k = rows * A(w.dim) * elem, v = rows * A(w.vdim) * elem;
+            if (!(md->cache[l] = md->take(fn, k * c.slots)) || !(md->values[l] = md->take(fn, v * c.slots)))
+                return false;
+            md->slot_bytes += k + v;
+        }
+        else if (w.mixer == LLAM_MIXER_DELTA)
+        {
+            const size_t state = (size_t)w.heads * P(w.dim) * P(w.vdim);
+            const size_t recent = (size_t)w.taps * (2 * w.kv_heads * P(w.dim) + w.heads * P(w.vdim));
+            if (!(md->memory[l] = (float *)md->take(fn, state * c.slots * 4)) || !(md->mem_m[l] = (float *)md->take(fn, recent * c.slots * 4)))
+                return false;
+            md->slot_bytes += (state + recent) * 4;
         }
         else
         {

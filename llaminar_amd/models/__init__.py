@@ -11,17 +11,24 @@ import json
 from pathlib import Path
 
 _FAMILIES = {}
+_SEQUENCE = set()   # families served by the sequence-model library alone
 
 
 class ConfigError(ValueError):
     """config.json does not describe a model of the family it names."""
 
 
-def register(name: str):
+def register(name: str, sequence: bool = False):
     def add(load):
         _FAMILIES[name] = load
+        if sequence:
+            _SEQUENCE.add(name)
         return load
     return add
+
+
+def needs_sequence_library(config: dict) -> bool:
+    return config["architecture"] in _SEQUENCE
 
 
 def families() -> list[str]:
@@ -58,4 +65,4 @@ def number(where: dict, key: str) -> float:
     return float(v)
 
 
-from . import dense, kogilix  # noqa: E402,F401  (each registers itself)
+from . import bosirax, dense, kogilix  # noqa: E402,F401  (each registers itself)

@@ -98,7 +98,7 @@ def weights(config: dict, tensors) -> ModelWeights:
                         layers=[layer(n) for n in range(len(layers))])
 
 
-@register("Kogilix")
+@register("Kogilix", sequence=True)
 def load(config: dict, model_dir: Path, slots: int = 8, cap: int = 4096, max_rows: int = 2048, dtype: str = "bfloat16",
          device_id: int = 0) -> SequenceModel:
     return SequenceModel(weights(config, SafeTensors(model_dir / "model.safetensors")), slots, cap, max_rows, dtype, device_id)

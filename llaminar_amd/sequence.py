@@ -1,8 +1,8 @@
 """ctypes door onto sequence models (include/llaminar_amd/sequence_model.h): layer descriptions,
 the weight layouts the kernels take, and the runner the engine steps.
 
-A model is described layer by layer (``LatentAttention`` or ``MatrixMemory``, then ``GatedFfn``,
-``Experts`` or nothing); which tensors hold the weights is the model family's business
+A model is described layer by layer (``LatentAttention``, ``GroupedAttention``, ``MatrixMemory`` or
+``DeltaRule``, then ``GatedFfn``, ``Experts`` or nothing); which tensors hold the weights is the model family's business
 (llaminar_amd/models).  Needs no PyTorch: device memory belongs to the library.
 """
 from __future__ import annotations
@@ -19,9 +19,9 @@ LIB_PATH = Path(__file__).resolve().parent / "lib" / "libllaminar_seq.so"
 
 BF16, F32 = 0, 1
 DTYPES = {"bfloat16": BF16, "float32": F32}
-OUT_F32, OUT_ADD, OUT_ELEM, OUT_GATED, OUT_RELU2 = range(5)
-MIXER_LATENT_ATTENTION, MIXER_MATRIX_MEMORY = 1, 2
-FFN_NONE, FFN_GATED, FFN_EXPERTS = 0, 1, 2
+OUT_F32, OUT_ADD, OUT_ELEM, OUT_GATED, OUT_RELU2, OUT_GATED_CLAMP = range(6)
+MIXER_LATENT_ATTENTION, MIXER_MATRIX_MEMORY, MIXER_ATTENTION, MIXER_DELTA = 1, 2, 3, 4
+FFN_NONE, FFN_GATED, FFN_EXPERTS, FFN_GATED_CLAMP = 0, 1, 2, 3
 
 
 class SequenceError(RuntimeError):
@@ -38,19 +38,28 @@ class Layer(ctypes.Structure):
                 ("w_in", c_void_p), ("w_out", c_void_p), ("q_rank", c_int), ("kv_rank", c_int), ("kv_from", c_int),
                 ("scale", c_float), ("q_norm", c_void_p), ("kv_norm", c_void_p), ("w_uq", c_void_p),
                 ("w_uk_t", c_void_p), ("w_uv", c_void_p), ("gate_cap", c_float), ("gate_bias", c_void_p),
-                ("head_norm", c_void_p), ("ffn", c_int), ("norm2", c_void_p), ("ff", c_int), ("w_up", c_void_p),
+                ("head_norm", c_void_p), ("kv_heads", c_int), ("rot_dims", c_int), ("chunk", c_int), ("turns", c_void_p),
+                ("taps", c_int), ("conv", c_void_p), ("a_log", c_void_p), ("dt_bias", c_void_p), ("parallel", c_int),
+                ("ffn", c_int), ("norm2", c_void_p), ("limit", c_float), ("ff", c_int), ("w_up", c_void_p),
                 ("w_down", c_void_p), ("experts", c_int), ("top", c_int), ("shared_ff", c_int), ("w_router", c_void_p),
                 ("router_bias", c_void_p), ("w_shared_up", c_void_p), ("w_shared_down", c_void_p)]
 
 
 class Globals(ctypes.Structure):
-    _fields_ = [("embed", c_void_p), ("final_norm", c_void_p), ("head", c_void_p)]
+    _fields_ = [("embed", c_void_p), ("final_norm", c_void_p), ("head", c_void_p), ("embed_scale", c_float),
+                ("pairs", c_void_p), ("buckets", c_int), ("mul_prev", c_long), ("mul_cur", c_long)]
 
 
 class LinearArgs(ctypes.Structure):
     _fields_ = [(n, c_void_p) for n in ("d_a", "d_w", "d_y", "d_bias", "d_norm", "d_h_out")] + \
                [("eps", c_float)] + [(n, c_int) for n in ("k_real", "M", "N", "K", "lda", "ldy", "out", "batch")] + \
-               [(n, c_long) for n in ("a_stride", "w_stride", "y_stride")]
+               [(n, c_long) for n in ("a_stride", "w_stride", "y_stride")] + [("limit", c_float)]
+
+
+class EmbedArgs(ctypes.Structure):
+    _fields_ = [("d_table", c_void_p), ("vocab", c_int), ("width", c_int), ("scale", c_float), ("d_pairs", c_void_p),
+                ("buckets", c_int), ("mul_prev", c_long), ("mul_cur", c_long)] + \
+               [(n, c_void_p) for n in ("d_row_slot", "d_row_pos", "d_history")] + [("cap", c_int)]
 
 
 class Entries(ctypes.Structure):
@@ -60,8 +69,20 @@ class Entries(ctypes.Structure):
 class MemoryArgs(ctypes.Structure):
     _fields_ = [("d_proj", c_void_p), ("ldp", c_int)] + \
                [(n, c_void_p) for n in ("d_gate_bias", "d_norm", "d_state", "d_m", "d_y")] + \
-               [(n, c_int) for n in ("heads", "dim", "vdim", "vdim_real")] + \
+               [(n, c_int) for n in ("ldy", "heads", "dim", "vdim", "vdim_real")] + \
                [(n, c_float) for n in ("q_scale", "gate_cap", "eps")]
+
+
+class AttentionArgs(ctypes.Structure):
+    _fields_ = [(n, c_int) for n in ("heads", "kv_heads", "dim", "vdim", "ring", "chunk")] + \
+               [("scale", c_float), ("d_k", c_void_p), ("d_v", c_void_p)]
+
+
+class DeltaArgs(ctypes.Structure):
+    _fields_ = [("d_proj", c_void_p), ("ldp", c_int)] + \
+               [(n, c_void_p) for n in ("d_conv", "d_a_log", "d_dt_bias", "d_norm", "d_state", "d_recent", "d_y")] + \
+               [(n, c_int) for n in ("ldy", "heads", "kv_heads", "dim", "vdim", "dim_real", "vdim_real", "taps")] + \
+               [("eps", c_float)]
 
 
 class ExpertsArgs(ctypes.Structure):
@@ -76,9 +97,21 @@ _I32P = POINTER(c_int32)
 # name -> (restype, argtypes); mirrors seq_api.h and sequence_model.h declaration by declaration
 SIGNATURES = {
     "llam_seq_linear": (c_bool, [POINTER(LinearArgs), c_int, c_int, c_void_p]),
-    "llam_seq_embed": (c_bool, [c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]),
+    "llam_seq_linear_pair": (c_bool, [POINTER(LinearArgs), POINTER(LinearArgs), c_int, c_int, c_void_p]),
+    "llam_seq_embed": (c_bool, [POINTER(EmbedArgs), c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]),
     "llam_seq_rmsnorm": (c_bool, [c_void_p, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p, c_int, c_int, c_int,
                                   c_int, c_void_p]),
+    "llam_seq_rmsnorm_pair": (c_bool, [c_void_p, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p, c_void_p, c_int, c_int,
+                                       c_int, c_int, c_void_p]),
+    "llam_seq_rotary": (c_bool, [POINTER(AttentionArgs), c_void_p, c_int, c_bool, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
+                                 c_int, c_int, c_int, c_void_p]),
+    "llam_seq_attention_scratch_floats": (c_size_t, [c_int]),
+    "llam_seq_attention": (c_bool, [POINTER(AttentionArgs), c_void_p, POINTER(Entries), c_int, c_int, c_int, c_int, c_void_p,
+                                    c_int, c_void_p, c_size_t, c_int, c_int, c_void_p]),
+    "llam_seq_delta_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int]),
+    "llam_seq_delta_decode": (c_bool, [POINTER(DeltaArgs), POINTER(Entries), c_int, c_int, c_int, c_int, c_void_p]),
+    "llam_seq_delta_prefill": (c_bool, [POINTER(DeltaArgs), POINTER(Entries), c_int, c_int, c_void_p, c_size_t, c_int, c_int,
+                                        c_void_p]),
     "llam_seq_latent_append": (c_bool, [c_void_p, c_int, c_void_p, c_float, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                         c_int, c_int, c_int, c_int, c_void_p]),
     "llam_seq_latent_scratch_floats": (c_size_t, [c_int, c_int, c_int, c_int, c_int]),
@@ -138,6 +171,11 @@ def P(n: int) -> int:
     return pad_to(n, 64)
 
 
+def A(n: int) -> int:
+    """Heads of the grouped-query attention are padded to 64, 128 or 256 (and may not be larger)."""
+    return 64 if n <= 64 else 128 if n <= 128 else 256
+
+
 def bf16_bits(x) -> np.ndarray:
     """float array -> bfloat16 bit patterns, to nearest even."""
     u = np.ascontiguousarray(x, dtype=np.float32).view(np.uint32)
@@ -157,14 +195,14 @@ def padded(w: np.ndarray, *shape: int) -> np.ndarray:
     return out
 
 
-def head_rows(w: np.ndarray, heads: int, dim: int) -> np.ndarray:
-    """[heads * dim, K] -> [heads * P(dim), K]: zero rows after each head's."""
-    return padded(w.reshape(heads, dim, -1), heads, P(dim), w.shape[1]).reshape(heads * P(dim), -1)
+def head_rows(w: np.ndarray, heads: int, dim: int, pad=P) -> np.ndarray:
+    """[heads * dim, K] -> [heads * pad(dim), K]: zero rows after each head's."""
+    return padded(w.reshape(heads, dim, -1), heads, pad(dim), w.shape[1]).reshape(heads * pad(dim), -1)
 
 
-def head_columns(w: np.ndarray, heads: int, dim: int) -> np.ndarray:
-    """[N, heads * dim] -> [N, heads * P(dim)]."""
-    return padded(w.reshape(-1, heads, dim), w.shape[0], heads, P(dim)).reshape(w.shape[0], -1)
+def head_columns(w: np.ndarray, heads: int, dim: int, pad=P) -> np.ndarray:
+    """[N, heads * dim] -> [N, heads * pad(dim)]."""
+    return padded(w.reshape(-1, heads, dim), w.shape[0], heads, pad(dim)).reshape(w.shape[0], -1)
 
 
 def tiled(w: np.ndarray) -> np.ndarray:
@@ -182,7 +220,7 @@ def gate_up_tiles(gate: np.ndarray, up: np.ndarray) -> np.ndarray:
 
 
 # ---- layer descriptions ----------------------------------------------------------------------------
-# Every tensor field is a bfloat16 bit pattern array in the orientation [out, in] (vectors [n]).
+# Every tensor field is a bfloat16 bit pattern array in the orientation [out, in] (vectors [n], norms also as float32).
 
 @dataclass
 class LatentAttention:
@@ -222,10 +260,50 @@ class MatrixMemory:
 
 
 @dataclass
+class GroupedAttention:
+    """Rotary attention, heads / kv_heads query heads on every key/value head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    turns: np.ndarray          # float64: revolutions per position of the rotated pairs
+    chunk: int | None          # positions see their own chunk only
+    kv_from: int | None
+    q: np.ndarray
+    k: np.ndarray | None
+    v: np.ndarray | None
+    out: np.ndarray
+
+
+@dataclass
+class DeltaRule:
+    """Gated delta rule, heads / kv_heads heads on every q/k head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    q: np.ndarray
+    q_conv: np.ndarray         # [channels, taps]
+    k: np.ndarray
+    k_conv: np.ndarray
+    v: np.ndarray
+    v_conv: np.ndarray
+    gate: np.ndarray
+    b: np.ndarray
+    a: np.ndarray
+    a_log: np.ndarray
+    dt_bias: np.ndarray
+    head_norm: np.ndarray      # [vdim], of all heads
+    out: np.ndarray
+
+
+@dataclass
 class GatedFfn:
     gate: np.ndarray
     up: np.ndarray
     down: np.ndarray
+    limit: float | None = None   # gelu(gate) * up, or with a limit the clamped activation of seq_api.h
 
 
 @dataclass
@@ -246,6 +324,17 @@ class LayerWeights:
     mixer: object
     norm2: np.ndarray | None = None
     ffn: object = None
+    parallel: bool = False   # mixer and feed-forward take the same x
+
+
+@dataclass
+class Pairs:
+    """Embedding of pairs of neighbouring tokens: row (previous * mul_prev + current * mul_cur) mod buckets of the
+    table, whose last row is for a sequence's first token."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+    table: np.ndarray
 
 
 @dataclass
@@ -258,6 +347,8 @@ class ModelWeights:
     head: np.ndarray
     layers: list = field(default_factory=list)   # of callables -> LayerWeights: a layer's host copies are
                                                  # made, uploaded and dropped one after the other
+    embed_scale: float = 1.0
+    pairs: Pairs | None = None
 
 
 def _i32(values) -> np.ndarray:
@@ -283,7 +374,11 @@ class SequenceModel:
         for n, make in enumerate(weights.layers):
             layer = self._layer(make())
             self._check(self.L.llam_seqm_set_layer(self.h, n, ctypes.byref(layer)))
-        g = Globals(self._raw(np.ascontiguousarray(weights.embed)), self._vector(weights.final_norm), self._matrix(weights.head))
+        g = Globals(self._raw(np.ascontiguousarray(weights.embed)), self._vector(weights.final_norm), self._matrix(weights.head),
+                    weights.embed_scale)
+        if weights.pairs is not None:
+            p = weights.pairs
+            g.pairs, g.buckets, g.mul_prev, g.mul_cur = self._raw(np.ascontiguousarray(p.table)), p.buckets, p.mul_prev, p.mul_cur
         self._check(self.L.llam_seqm_set_globals(self.h, ctypes.byref(g)))
 
     # -- weights
@@ -297,14 +392,20 @@ class SequenceModel:
         return self._raw(tiled(w))
 
     def _vector(self, bits: np.ndarray, *shape: int) -> int:
-        v = bf16_to_f32(bits)
+        v = bits if bits.dtype == np.float32 else bf16_to_f32(bits)
         return self._raw(np.ascontiguousarray(padded(v, *(shape or (P(v.shape[0]),)))))
 
     def _layer(self, w: LayerWeights) -> Layer:
         out = Layer(norm1=self._vector(w.norm1))
         m = w.mixer
         out.heads, out.dim, out.vdim, out.kv_from = m.heads, m.dim, m.vdim, -1
-        out.w_out = self._matrix(padded(head_columns(m.out, m.heads, m.vdim), P(self.width), m.heads * P(m.vdim)))
+        pad = A if isinstance(m, GroupedAttention) else P
+        w_out = padded(head_columns(m.out, m.heads, m.vdim, pad), P(self.width), m.heads * pad(m.vdim))
+        out.parallel = w.parallel and w.ffn is not None
+        if out.parallel:
+            down = w.ffn.down
+            w_out = np.concatenate([w_out, padded(down, P(self.width), P(down.shape[1]))], axis=1)
+        out.w_out = self._matrix(w_out)
         if isinstance(m, LatentAttention):
             out.mixer = MIXER_LATENT_ATTENTION
             out.q_rank, out.kv_rank, out.scale = m.q_rank, m.kv_rank, m.scale
@@ -328,6 +429,25 @@ class SequenceModel:
                                                     m.i, m.f]))
             out.gate_bias = self._vector(np.concatenate([m.i_bias, m.f_bias]), 2 * m.heads)
             out.head_norm = self._vector(m.head_norm.reshape(m.heads, m.vdim), m.heads, P(m.vdim))
+        elif isinstance(m, GroupedAttention):
+            out.mixer, out.kv_heads, out.scale, out.chunk = MIXER_ATTENTION, m.kv_heads, m.scale, m.chunk or 0
+            out.kv_from = -1 if m.kv_from is None else m.kv_from
+            rows = [head_rows(m.q, m.heads, m.dim, A)]
+            if m.kv_from is None:
+                rows += [head_rows(m.k, m.kv_heads, m.dim, A), head_rows(m.v, m.kv_heads, m.vdim, A)]
+            out.w_in = self._matrix(np.concatenate(rows))
+            out.rot_dims = 2 * len(m.turns)
+            if out.rot_dims:
+                out.turns = self._raw(np.ascontiguousarray(m.turns, dtype=np.float64))
+        elif isinstance(m, DeltaRule):
+            out.mixer, out.kv_heads, out.taps = MIXER_DELTA, m.kv_heads, m.q_conv.shape[1]
+            out.w_in = self._matrix(np.concatenate([head_rows(m.q, m.kv_heads, m.dim), head_rows(m.k, m.kv_heads, m.dim),
+                                                    head_rows(m.v, m.heads, m.vdim), head_rows(m.gate, m.heads, m.vdim), m.b, m.a]))
+            taps = np.concatenate([head_rows(m.q_conv, m.kv_heads, m.dim), head_rows(m.k_conv, m.kv_heads, m.dim),
+                                   head_rows(m.v_conv, m.heads, m.vdim)])
+            out.conv = self._vector(np.ascontiguousarray(taps.T), *taps.T.shape)
+            out.a_log, out.dt_bias = self._vector(m.a_log, m.heads), self._vector(m.dt_bias, m.heads)
+            out.head_norm = self._vector(m.head_norm)
         else:
             raise TypeError(f"mixer {type(m).__name__}")
         f = w.ffn
@@ -335,9 +455,11 @@ class SequenceModel:
             return out
         out.norm2 = self._vector(w.norm2)
         if isinstance(f, GatedFfn):
-            out.ffn, out.ff = FFN_GATED, f.gate.shape[0]
+            out.ffn, out.ff = FFN_GATED if f.limit is None else FFN_GATED_CLAMP, f.gate.shape[0]
+            out.limit = f.limit or 0.0
             out.w_up = self._raw(gate_up_tiles(f.gate, f.up))
-            out.w_down = self._matrix(padded(f.down, P(self.width), P(out.ff)))
+            if not out.parallel:
+                out.w_down = self._matrix(padded(f.down, P(self.width), P(out.ff)))
         elif isinstance(f, Experts):
             out.ffn, out.ff, out.experts, out.top = FFN_EXPERTS, f.up[0].shape[0], len(f.up), f.top
             ff, wp = P(out.ff), P(self.width)

@@ -133,5 +133,5 @@ def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap
     head, b = matrix(vocab, P(width))
     model.weight_bytes.append(b)
     torch.cuda.synchronize()
-    model._check(model.L.llam_seqm_set_globals(model.h, ctypes.byref(sq.Globals(embed.data_ptr(), vector(P(width)), head))))
+    model._check(model.L.llam_seqm_set_globals(model.h, ctypes.byref(sq.Globals(embed.data_ptr(), vector(P(width)), head, 1.0))))
     return model

@@ -54,7 +54,7 @@ def main(argv=None) -> int:
     from . import build, models
     from .engine import Engine
 
-    if models.read_config(args.model)["architecture"] == "Kogilix":
+    if models.needs_sequence_library(models.read_config(args.model)):
         build.build_seq(force=False, verbose=False)
     out = Path(args.out)
     out.mkdir(parents=True, exist_ok=True)
