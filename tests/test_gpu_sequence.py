@@ -14,6 +14,7 @@ from llaminar_amd.engine import Engine
 from llaminar_amd.models import kogilix
 from oracle import sequence_oracle as so
 from tests import sequence_models as sm
+from tests.sequence_models import check, run, tokens_of
 
 pytestmark = pytest.mark.gpu
 ROOT = Path(__file__).resolve().parent.parent
@@ -27,32 +28,6 @@ def one_runtime(dev):
 
 def load(cfg, tensors, dtype="float32", slots=4, cap=640, max_rows=640):
     return sequence.SequenceModel(kogilix.weights(cfg, tensors), slots, cap, max_rows, dtype)
-
-
-def run(model, slot, tokens, cuts, at=0):
-    """Logits of every token, fed in the given portions."""
-    rows = []
-    for n in cuts:
-        rows.append(model.forward([(slot, at, tokens[at:at + n])], range(n)))
-        at += n
-    return np.concatenate(rows)
-
-
-def tokens_of(cfg, n, seed=0):
-    return np.random.default_rng(seed + 1000).integers(0, cfg["vocab"], n).tolist()
-
-
-def check(got, want, dtype, f32=2e-5, bf16=0.02, note=""):
-    e = sm.row_errors(got, want)
-    print(f"[sequence] {note} {dtype}: worst {e.max():.2e} median {np.median(e):.2e}", flush=True)
-    if dtype == "float32":
-        # where a memory's output nearly cancels, the norm behind it magnifies the last bits (weights changed by half
-        # a 32-bit rounding move such rows by 1e-5): a few rows may be further off, a wrong one is off by 1e-2
-        ok = np.median(e) < f32 / 5 and np.mean(e > f32) <= 0.05 and e.max() < 30 * f32
-        assert ok, (note, int(e.argmax()), float(e.max()), float(np.median(e)))
-    else:
-        # a router may choose otherwise where two logits are within a bfloat16 rounding: a few rows
-        assert np.median(e) < bf16 and np.mean(e > 4 * bf16) <= 0.05, (note, int(e.argmax()), float(e.max()), float(np.median(e)))
 
 
 MECHANISMS = {

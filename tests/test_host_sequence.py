@@ -9,7 +9,7 @@ import numpy as np
 import pytest
 
 from llaminar_amd import engine, models, safetensors_io, sequence, trace
-from llaminar_amd.models import kogilix
+from llaminar_amd.models import bosirax, kogilix
 from oracle import sequence_oracle as so
 from tests import sequence_models as sm
 
@@ -48,6 +48,23 @@ def test_bad_arguments_are_refused_before_any_launch():
     assert not lib.llam_seq_experts(ctypes.byref(x), 1, p, 1 << 30, 0, 0, None) and "top=5" in err()
     assert not lib.llam_seq_latent_attention(p, p, ctypes.byref(e), 0, 1, 1, 65, 1, 64, 64, 1.0, p, p, 1 << 30, 0, 0, None)
     assert "max_len=65" in err()
+    g = sequence.AttentionArgs(5, 2, 64, 64, 128, 0, 1.0, p, p)
+    assert not lib.llam_seq_attention(ctypes.byref(g), p, ctypes.byref(e), 0, 1, 1, 65, p, 320, p, 1 << 30, 0, 0, None) and "kv_heads" in err()
+    g = sequence.AttentionArgs(4, 2, 96, 64, 128, 0, 1.0, p, p)
+    assert not lib.llam_seq_attention(ctypes.byref(g), p, ctypes.byref(e), 0, 1, 1, 65, p, 256, p, 1 << 30, 0, 0, None) and "padded" in err()
+    g = sequence.AttentionArgs(4, 2, 64, 64, 128, 0, 1.0, p, p)
+    assert not lib.llam_seq_attention(ctypes.byref(g), p, ctypes.byref(e), 0, 1, 1, 129, p, 256, p, 1 << 30, 0, 0, None) and "129 positions" in err()
+    assert not lib.llam_seq_rotary(ctypes.byref(g), p, 256, True, p, 4, p, p, p, 1, 0, 0, None) and "ldp=256" in err()
+    d = sequence.DeltaArgs(d_proj=p, ldp=4096, d_conv=p, d_a_log=p, d_dt_bias=p, d_norm=p, d_state=p, d_recent=p, d_y=p, ldy=64, heads=1,
+                           kv_heads=1, dim=320, vdim=64, dim_real=300, vdim_real=64, taps=4, eps=1e-5)
+    assert not lib.llam_seq_delta_decode(ctypes.byref(d), ctypes.byref(e), 0, 1, 0, 0, None) and "256" in err()
+    d.dim, d.dim_real, d.taps = 64, 64, 0
+    assert not lib.llam_seq_delta_prefill(ctypes.byref(d), ctypes.byref(e), 0, 5, p, 1 << 30, 0, 0, None) and "taps=0" in err()
+    m = sequence.EmbedArgs(d_table=p, vocab=9, width=64, scale=1.0, d_pairs=p, buckets=0)
+    assert not lib.llam_seq_embed(ctypes.byref(m), p, p, 1, 64, 0, None) and "buckets=0" in err()
+    a = sequence.LinearArgs(d_a=p, d_w=p, d_y=p, M=1, N=16, K=64, lda=64, ldy=16, batch=1)
+    b = sequence.LinearArgs(d_a=p, d_w=p, d_y=p, M=1, N=16, K=128, lda=128, ldy=16, batch=1)
+    assert not lib.llam_seq_linear_pair(ctypes.byref(a), ctypes.byref(b), 0, 0, None) and "same rows" in err()
     assert not lib.llam_seqm_create(ctypes.byref(sequence.Config(0, 1, 1, 1, 1, 1, 0, 1e-5, 0)))
 
 
@@ -112,7 +129,8 @@ def test_safetensors_round_trip_and_refusals(tmp_path):
 # ---- configuration -----------------------------------------------------------------------------------
 
 def test_registry_names_the_families(tmp_path):
-    assert {"Kogilix", "DenseQ4K"} <= set(models.families())
+    assert {"Kogilix", "Bosirax", "DenseQ4K"} <= set(models.families())
+    assert [models.needs_sequence_library({"architecture": n}) for n in ("Bosirax", "Kogilix", "DenseQ4K")] == [True, True, False]
     (tmp_path / "config.json").write_text('{"architecture": "Nobody"}')
     with pytest.raises(models.ConfigError, match="Nobody"):
         models.load_model(tmp_path)
@@ -149,6 +167,50 @@ def test_faulty_configurations_are_refused(spoil):
     with pytest.raises((models.ConfigError, AssertionError)) as e:
         [make() for make in kogilix.weights(cfg, tensors).layers]
     assert e.type is models.ConfigError
+
+
+def test_every_branch_of_the_bosirax_configuration_is_read():
+    cfg = sm.bosirax(sm.delta(mlp=sm.clamped(limit=1.25)), sm.attention(chunk=9, stretch=sm.scaling()), sm.attention(kv_from=1, heads=6, scale=0.5, mlp=sm.clamped(ff=50)),
+                     sm.attention(rot=0))
+    w = bosirax.weights(cfg, sm.random_bosirax(cfg))
+    a, b, c, d = [make() for make in w.layers]
+    assert w.embed_scale == 1.7 and (w.pairs.buckets, w.pairs.mul_prev, w.pairs.mul_cur, len(w.pairs.table)) == (97, 13, 5, 98)
+    assert all(x.parallel for x in (a, b, c, d)) and a.norm1.dtype == np.float32 and abs(a.norm1.mean() - 1) < 0.2
+    assert a.mixer.q_conv.shape == (80, 4) and a.mixer.v_conv.shape == (96, 4) and a.ffn.limit == 1.25 and a.mixer.head_norm.shape == (24,)
+    assert b.ffn is None and b.norm2 is None and b.mixer.chunk == 9 and len(b.mixer.turns) == 6 and b.mixer.k.shape == (48, 136)
+    assert c.mixer.k is None and c.mixer.v is None and c.mixer.kv_from == 1 and c.mixer.heads == 6 and c.mixer.chunk is None
+    assert len(d.mixer.turns) == 0
+    cfg["embedding"].pop("bigram")
+    assert bosirax.weights(cfg, sm.random_bosirax(cfg)).pairs is None
+
+
+@pytest.mark.parametrize("spoil", [
+    lambda c: c["layers"][1]["mixer"].update(kv_from=1), lambda c: c["layers"][1]["mixer"].update(kv_from=3),
+    lambda c: c["layers"][3]["mixer"].update(kv_from=2), lambda c: c["layers"][3]["mixer"].update(kv_from=1),
+    lambda c: c["layers"][1]["mixer"].update(kv_heads=1), lambda c: c["layers"][0]["mixer"].update(kv_heads=3),
+    lambda c: c["layers"][0]["mixer"]["rot"].update(dims=3), lambda c: c["layers"][0]["mixer"]["rot"].update(dims=26),
+    lambda c: c["layers"][0]["mixer"]["rot"].update(scaling={"factor": 2.0}), lambda c: c["layers"][0]["mixer"].pop("rot"),
+    lambda c: c["layers"][0]["mixer"].update(mask={"size": 0}), lambda c: c["layers"][2]["mixer"].update(conv=0),
+    lambda c: c["layers"][2].update(mlp={"kind": "moe"}), lambda c: c["layers"][2]["mlp"].pop("limit"),
+    lambda c: c["layers"][2].update(type="mlstm"), lambda c: c.pop("embedding"), lambda c: c["embedding"]["bigram"].update(buckets=0)])
+def test_faulty_bosirax_configurations_are_refused(spoil):
+    cfg = sm.bosirax(sm.attention(), sm.attention(kv_from=0), sm.delta(mlp=sm.clamped()), sm.attention(kv_from=0))
+    tensors = sm.random_bosirax(cfg)
+    spoil(cfg)
+    with pytest.raises((models.ConfigError, AssertionError)) as e:
+        [make() for make in bosirax.weights(cfg, tensors).layers]
+    assert e.type is models.ConfigError
+
+
+@pytest.mark.parametrize("stretch", [None, sm.scaling(), sm.scaling(8.0, 1.5, 6.0, 300)])
+def test_rotary_turns_are_the_plain_frequencies(stretch):
+    rot = dict(dims=46, base=700.0)
+    if stretch:
+        rot["scaling"] = stretch
+        wave = 2 * np.pi / so.rotary_frequencies(46, 700.0)
+        bands = {(w > stretch["original"] / stretch["low"]) - int(w < stretch["original"] / stretch["high"]) for w in wave}
+        assert bands == {-1, 0, 1}
+    assert np.allclose(bosirax.rotary_turns(rot) * 2 * np.pi, so.rotary_frequencies(46, 700.0, stretch), rtol=1e-13)
 
 
 # ---- scheduler -----------------------------------------------------------------------------------------
@@ -282,3 +344,49 @@ def test_latent_attention_is_causal():
     tokens = [5, 9, 100, 7, 3]
     a, b = so.kogilix(cfg, t, tokens), so.kogilix(cfg, t, tokens[:3] + [1, 2])
     assert np.array_equal(a[:3], b[:3]) and not np.allclose(a[3], b[3])
+
+
+def test_rotation_keeps_lengths_and_sees_distances():
+    rng = np.random.default_rng(4)
+    freq = so.rotary_frequencies(6, 100.0)
+    x = rng.standard_normal((2, 1, 8))
+    y = so.rotate(x, [3, 3], freq)
+    assert np.allclose(np.linalg.norm(y, axis=-1), np.linalg.norm(x, axis=-1)) and np.array_equal(y[..., 6:], x[..., 6:])
+    dots = [so.rotate(x[:1], [p + 5], freq)[0, 0] @ so.rotate(x[1:], [p], freq)[0, 0] for p in (0, 7, 100)]
+    assert np.allclose(dots, dots[0])
+
+
+def test_delta_recurrence_equals_its_chunked_form():
+    """The triangular system of a chunk, solved at once, against the recurrence token by token."""
+    rng = np.random.default_rng(3)
+    T, d, v = 19, 6, 5
+    q, k, val = so.unit(rng.standard_normal((T, d))), so.unit(rng.standard_normal((T, d))), rng.standard_normal((T, v))
+    decay, beta = rng.uniform(0.5, 1.0, T), rng.uniform(0.0, 1.0, T)
+    o, S = so.delta_recurrence(q, k, val, decay, beta)
+    G = np.cumsum(np.log(decay))
+    f = np.tril(np.exp(G[:, None] - G[None]))
+    u = np.linalg.solve(np.eye(T) + np.tril(beta[:, None] * f * (k @ k.T), -1), beta[:, None] * val)
+    assert np.allclose((f * (q @ k.T)) @ u, o) and np.allclose((np.exp(G[-1] - G)[:, None] * k).T @ u, S)
+
+
+def test_delta_rule_replaces_what_a_key_held():
+    k = np.eye(3)[[0, 1, 0]]
+    v = np.array([[1.0, 2.0], [3.0, 4.0], [5.0, 6.0]])
+    o, S = so.delta_recurrence(k, k, v, np.ones(3), np.ones(3))
+    assert np.allclose(S, [[5, 6], [3, 4], [0, 0]]) and np.allclose(o, v)
+
+
+def test_chunked_attention_forgets_at_the_edge():
+    rng = np.random.default_rng(8)
+    q, k, v = (rng.standard_normal((9, 2, 4)) for _ in range(3))
+    o = so.grouped_attention(q, k, v, 0.5, 4)
+    assert np.allclose(o[4], v[4]) and np.allclose(o[8], v[8])
+    assert np.allclose(o[4:8], so.grouped_attention(q[4:8], k[4:8], v[4:8], 0.5, None))
+
+
+def test_short_convolution_and_pairs():
+    x = np.arange(1.0, 6.0)[:, None]
+    y = so.short_convolution(x, np.array([[100.0, 10.0, 1.0]]))
+    z = np.array([1, 12, 123, 234, 345.0])[:, None]
+    assert np.allclose(y, z * so.sigmoid(z))
+    assert so.bigram_rows([3, 1, 4], 10, 1, 7) == [7, 31 % 7, 14 % 7]
