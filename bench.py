@@ -370,24 +370,17 @@ def bench_decode(args, torch, capi, synth, dev):
 
 
 SEQUENCE_SIZES = {
-    # width, dense ff, experts (count, top, ff, shared ff), latent (heads, dim, vdim, q_rank, kv_rank), memory (heads, dim, vdim), and the
-    # quantized dense model of the same width, feed-forward width and number of layers
     "2048": dict(width=2048, ff=8192, moe=(64, 6, 1408, 2816), latent=(16, 128, 128, 768, 512), memory=(4, 256, 512),
-                 dense=dict(hidden=2048, n_heads=32, n_kv=4, ffn=8192)),
+                 attention=(16, 4, 128, 128), delta=(16, 8, 128, 128), dense=dict(hidden=2048, n_heads=32, n_kv=4, ffn=8192)),
     "5120": dict(width=5120, ff=25600, moe=(64, 6, 1536, 3072), latent=(64, 128, 128, 1536, 512), memory=(8, 256, 512),
-                 dense=dict(hidden=5120, n_heads=64, n_kv=8, ffn=25600)),
+                 attention=(40, 8, 128, 128), delta=(40, 20, 128, 128), dense=dict(hidden=5120, n_heads=64, n_kv=8, ffn=25600)),
 }
+SEQUENCE_VOCAB = 32768
 
 
-def bench_sequence(args, torch, capi, synth, dev):
-    """Sequence model of four layers (memory + gated, latent attention + experts, memory + experts, latent
-    attention on the second layer's cache + gated) over random bf16 weights: prefill of a 2048-token portion and greedy
-    decoding at the given context, beside the quantized dense decoder of the same width, feed-forward width, depth
-    and vocabulary (whose step has no prefill: its prompts run token by token)."""
-    from llaminar_amd import sequence as sq
-    from llaminar_amd.decoder import DenseDecoder, Shape
-
-    def layer(z, mixer, ffn, kv_from=-1):
+def _kogilix_layers(sq, z):
+    """memory + gated, latent attention + experts, memory + experts, latent attention on the second layer's cache + gated"""
+    def layer(mixer, ffn, kv_from=-1):
         w = sq.Layer(mixer=mixer, kv_from=kv_from, ffn=ffn)
         if mixer == sq.MIXER_LATENT_ATTENTION:
             w.heads, w.dim, w.vdim, w.q_rank, w.kv_rank = z["latent"]
@@ -399,44 +392,89 @@ def bench_sequence(args, torch, capi, synth, dev):
             w.experts, w.top, w.ff, w.shared_ff = z["moe"]
         return w
 
-    vocab, ctx, B, portion = 32768, args.context, args.batch, 2048
+    LAT, MEM, GATED, EXPERTS = sq.MIXER_LATENT_ATTENTION, sq.MIXER_MATRIX_MEMORY, sq.FFN_GATED, sq.FFN_EXPERTS
+    return [layer(MEM, GATED), layer(LAT, EXPERTS), layer(MEM, EXPERTS), layer(LAT, GATED, kv_from=1)]
+
+
+def _bosirax_layers(sq, z):
+    """delta rule, grouped-query attention in chunks of 8192, attention on the second layer's cache, delta rule; every
+    layer parallel with a clamped gated feed-forward"""
+    def layer(mixer, kv_from=-1):
+        w = sq.Layer(mixer=mixer, kv_from=kv_from, parallel=1, ffn=sq.FFN_GATED_CLAMP, ff=z["ff"], limit=7.0)
+        w.heads, w.kv_heads, w.dim, w.vdim = z["attention" if mixer == sq.MIXER_ATTENTION else "delta"]
+        w.chunk, w.taps = 8192, 4
+        return w
+
+    return [layer(sq.MIXER_DELTA), layer(sq.MIXER_ATTENTION), layer(sq.MIXER_ATTENTION, kv_from=1), layer(sq.MIXER_DELTA)]
+
+
+SEQUENCE_FAMILIES = {"kogilix": _kogilix_layers, "bosirax": _bosirax_layers}
+
+
+def _state_bytes(sq, w, ctx):
+    """Bytes of cache and state one sequence's decode step reads and writes in a layer."""
+    if w.mixer == sq.MIXER_LATENT_ATTENTION:
+        return ctx * w.kv_rank * 2
+    if w.mixer == sq.MIXER_ATTENTION:
+        return min(ctx, w.chunk) * w.kv_heads * (w.dim + w.vdim) * 2
+    return w.heads * sq.P(w.dim) * (sq.P(w.vdim) + (16 if w.mixer == sq.MIXER_MATRIX_MEMORY else 0)) * 8
+
+
+def _sequence_row(args, torch, synth, sq, dev, family, z, steps):
+    """Prefill of a 2048-token portion and greedy decoding of one family at one size."""
+    vocab, ctx, B, portion = SEQUENCE_VOCAB, args.context, args.batch, 2048
+    layers = SEQUENCE_FAMILIES[family](sq, z)
+    cap = ctx + steps + args.warmup + 16
+    model = synth.sequence_model_torch(layers, z["width"], vocab, dev, slots=B, cap=cap, max_rows=portion,
+                                       pairs=100003 if family == "bosirax" else 0)
+    ids = torch.randint(0, vocab, (portion,), generator=torch.Generator().manual_seed(1)).numpy()
+    for slot in range(B):   # the context every decode step finds
+        for at in range(0, ctx, portion):
+            model.forward([(slot, at, ids[:min(portion, ctx - at)])])
+    row = {"family": family, "width": z["width"], "batch": B, "context": ctx, "layers": len(layers)}
+    if args.phase in ("prefill", "both"):
+        reps = max(3, min(20, args.steps // 10))
+        for at, key in ((0, "prefill_ms_first_portion"), (ctx - portion, "prefill_ms_last_portion")):
+            if at < 0:
+                continue
+            t0 = time.perf_counter()
+            for _ in range(reps):
+                model.forward([(0, at, ids)], [portion - 1], best=True)
+            row[key] = round((time.perf_counter() - t0) * 1e3 / reps, 3)
+        row["prefill_tokens_per_s"] = round(portion * 1e3 / row["prefill_ms_first_portion"], 1)
+    if args.phase in ("decode", "both"):
+        pos, slots, tok = [ctx] * B, list(range(B)), [1] * B
+        model.decode(slots, pos, tok, max(args.warmup, 2))
+        model.decode(slots, pos, tok, steps)
+        row["decode_ms"] = round(model.last_decode_ms / steps, 4)
+        row["decode_tokens_per_s"] = round(B * 1e3 / row["decode_ms"], 1)
+        row["weight_bytes_batch1"] = sum(model.weight_bytes)
+        row["state_bytes_per_step"] = B * sum(_state_bytes(sq, w, ctx) for w in layers)
+        row["hbm_frac_batch1_bytes"] = round((row["weight_bytes_batch1"] + row["state_bytes_per_step"]) / (row["decode_ms"] * 1e-3) / 8e12, 4)
+    model.close()
+    del model
+    torch.cuda.empty_cache()
+    return row
+
+
+def bench_sequence(args, torch, capi, synth, dev):
+    """Sequence models of four layers over random bf16 weights: prefill of a 2048-token portion and greedy decoding at the
+    given context.  kogilix: beside the quantized dense decoder of the same width, feed-forward width, depth and
+    vocabulary (whose step has no prefill: its prompts run token by token).  bosirax: beside kogilix of the same width."""
+    from llaminar_amd import sequence as sq
+    from llaminar_amd.decoder import DenseDecoder, Shape
+
+    ctx, B = args.context, args.batch
     steps, rows = max(args.steps, 20), []
+    cap = ctx + steps + args.warmup + 16
     for name in args.sizes.split(","):
         z = SEQUENCE_SIZES[name]
-        LAT, MEM, GATED, EXPERTS = sq.MIXER_LATENT_ATTENTION, sq.MIXER_MATRIX_MEMORY, sq.FFN_GATED, sq.FFN_EXPERTS
-        layers = [layer(z, MEM, GATED), layer(z, LAT, EXPERTS), layer(z, MEM, EXPERTS), layer(z, LAT, GATED, kv_from=1)]
-        cap = ctx + steps + args.warmup + 16
-        model = synth.sequence_model_torch(layers, z["width"], vocab, dev, slots=B, cap=cap, max_rows=portion)
-        ids = torch.randint(0, vocab, (portion,), generator=torch.Generator().manual_seed(1)).numpy()
-        for slot in range(B):   # the context every decode step finds
-            for at in range(0, ctx, portion):
-                model.forward([(slot, at, ids[:min(portion, ctx - at)])])
-        row = {"width": z["width"], "batch": B, "context": ctx, "layers": 4}
-        if args.phase in ("prefill", "both"):
-            reps = max(3, min(20, args.steps // 10))
-            for at, key in ((0, "prefill_ms_first_portion"), (ctx - portion, "prefill_ms_last_portion")):
-                if at < 0:
-                    continue
-                t0 = time.perf_counter()
-                for _ in range(reps):
-                    model.forward([(0, at, ids)], [portion - 1], best=True)
-                row[key] = round((time.perf_counter() - t0) * 1e3 / reps, 3)
-            row["prefill_tokens_per_s"] = round(portion * 1e3 / row["prefill_ms_first_portion"], 1)
-        if args.phase in ("decode", "both"):
-            pos, slots, tok = [ctx] * B, list(range(B)), [1] * B
-            model.decode(slots, pos, tok, max(args.warmup, 2))
-            model.decode(slots, pos, tok, steps)
-            row["decode_ms"] = round(model.last_decode_ms / steps, 4)
-            row["decode_tokens_per_s"] = round(B * 1e3 / row["decode_ms"], 1)
-            row["weight_bytes_batch1"] = sum(model.weight_bytes)
-            row["state_bytes_per_step"] = B * (2 * sum(w.heads * sq.P(w.dim) * (sq.P(w.vdim) + 16) * 8 for w in layers[:1]) +
-                                               2 * ctx * layers[1].kv_rank * 2)
-            row["hbm_frac_batch1_bytes"] = round((row["weight_bytes_batch1"] + row["state_bytes_per_step"]) / (row["decode_ms"] * 1e-3) / 8e12, 4)
-        model.close()
-        del model
-        torch.cuda.empty_cache()
-        if args.phase in ("decode", "both") and not args.no_decode:
-            shape = Shape(n_layers=4, vocab=vocab, **z["dense"])
+        row = _sequence_row(args, torch, synth, sq, dev, args.family, z, steps)
+        if args.family != "kogilix":
+            if not args.no_decode:
+                row["beside"] = _sequence_row(args, torch, synth, sq, dev, "kogilix", z, steps)
+        elif args.phase in ("decode", "both") and not args.no_decode:
+            shape = Shape(n_layers=4, vocab=SEQUENCE_VOCAB, **z["dense"])
             dec = DenseDecoder(shape, B, (cap + 31) // 32 * 32, dev, seed=11)
             dec.set_state([1] * B, [ctx - 1] * B)
             stream = torch.cuda.Stream()
@@ -533,9 +571,9 @@ def parse():
                     help="layer: the headline decode-layer step (default); gemm: prefill int8 GEMM 512x25600x5120 Q4_K; "
                          "moe: 256-expert top-8 IQ3_S expert FFN decode; gemv: single GEMVs of every format and layer shape; "
                          "read-order: read-only probes of the GEMV's load stream in several orders; "
-                         "sequence: prefill and decoding of a sequence model (latent attention, matrix memory, experts; bf16 weights) "
-                         "beside the quantized dense decoder of the same width")
+                         "sequence: prefill and decoding of a sequence model (--family; bf16 weights) beside the closest other model of the same width")
     ap.add_argument("--sizes", default="2048,5120", help="sequence workload: widths, with commas between them")
+    ap.add_argument("--family", choices=sorted(SEQUENCE_FAMILIES), default="kogilix", help="sequence workload: the model")
     ap.add_argument("--phase", choices=["prefill", "decode", "both"], default="both", help="sequence workload: what is timed")
     ap.add_argument("--batch", type=int, default=1, help="activation rows / tokens per step")
     ap.add_argument("--layers", type=int, default=4, help="distinct weight sets rotated through")

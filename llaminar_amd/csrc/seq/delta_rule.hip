@@ -52,13 +52,24 @@ namespace llamql
         f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
         const int taps = p.a.taps;
         const float *recent = p.a.d_recent + (size_t)slot * taps * p.channels;
-        for (int j = 0; j < taps; ++j)
+        const int place = pos % taps;
+        for (int b0 = 0; b0 < taps; b0 += 4) // (four taps at a time, their inputs all requested before the first is used)
         {
-            const int back = taps - 1 - j, at = pos - back;
-            if (at < 0)
-                continue;
-            const float *x = at >= pos0 ? p.a.d_proj + (size_t)(r - back) * p.a.ldp : recent + (size_t)(at % taps) * p.channels;
-            y = y + *reinterpret_cast<const f32x4 *>(p.a.d_conv + (size_t)j * p.channels + ch) * *reinterpret_cast<const f32x4 *>(x + ch);
+            f32x4 x[4], w[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+            {
+                const int back = b0 + i < taps ? b0 + i : taps - 1, at = pos - back;
+                const float *row = at >= pos0 ? p.a.d_proj + (size_t)(r - back) * p.a.ldp
+                                              : recent + (size_t)(back <= place ? place - back : place - back + taps) * p.channels;
+                x[i] = *reinterpret_cast<const f32x4 *>(row + ch);
+                w[i] = *reinterpret_cast<const f32x4 *>(p.a.d_conv + (size_t)(taps - 1 - back) * p.channels + ch);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int k = 0; k < 4; ++k) // before the sequence's start there is nothing, whatever the state holds
+                    y[k] += b0 + i < taps && pos >= b0 + i ? w[i][k] * x[i][k] : 0.0f;
         }
 #pragma unroll
         for (int i = 0; i < 4; ++i)
@@ -66,9 +77,13 @@ namespace llamql
         return y;
     }
 
-    __device__ __forceinline__ float delta_unit(f32x4 y) // of a wavefront's vector: the factor that makes it a unit vector
+    // the factor that makes a vector a unit vector, four of its values in each of `lanes` neighbouring lanes
+    __device__ __forceinline__ float delta_unit(f32x4 y, int lanes)
     {
-        return 1.0f / sqrtf(wave_sum64(y[0] * y[0] + y[1] * y[1] + y[2] * y[2] + y[3] * y[3]) + 1e-6f);
+        float sum = y[0] * y[0] + y[1] * y[1] + y[2] * y[2] + y[3] * y[3];
+        for (int off = lanes / 2; off > 0; off >>= 1)
+            sum += __shfl_xor(sum, off, 64);
+        return 1.0f / sqrtf(sum + 1e-6f);
     }
 
     // ---- decoding -------------------------------------------------------------------------------
@@ -111,7 +126,7 @@ namespace llamql
             f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
             if (lane * 4 < dim)
                 y = delta_conv(p, r, pos, pos, slot, ch);
-            y = y * (delta_unit(y) * (wave == 0 ? 1.0f / sqrtf((float)a.dim_real) : 1.0f));
+            y = y * (delta_unit(y, 64) * (wave == 0 ? 1.0f / sqrtf((float)a.dim_real) : 1.0f));
             if (lane * 4 < dim)
             {
                 *reinterpret_cast<f32x4 *>((wave == 0 ? s_q : s_k) + lane * 4) = y;
@@ -201,31 +216,40 @@ namespace llamql
     }
 
     // ---- prompts: convolutions, unit vectors, gates -------------------------------------------------
-    // A wavefront per token and vector: q heads, k heads, v heads.
+    // Workgroup = INPUT_TOKENS neighbouring tokens of one vector (q heads, k heads, v heads), 16, 32 or 64 lanes
+    // per token: a token's inputs are used by the next ones' taps while they are near.
+    constexpr int INPUT_TOKENS = 16;
     __global__ void __launch_bounds__(256)
         delta_inputs_kernel(DeltaArgs p)
     {
         const llam_seq_delta_args &a = p.a;
-        const int lane = threadIdx.x & 63, e = p.entry, t = blockIdx.y;
-        const int unit = blockIdx.x * 4 + (threadIdx.x >> 6), G = a.kv_heads;
-        const int r = p.row0[e] + t, slot = p.slot[e], pos0 = p.pos[e];
-        if (unit < 2 * G)
+        const int e = p.entry, n = p.ntok[e], unit = blockIdx.x, G = a.kv_heads;
+        const int slot = p.slot[e], pos0 = p.pos[e];
+        const int size = unit < 2 * G ? a.dim : a.vdim, lanes = size <= 64 ? 16 : size <= 128 ? 32 : 64;
+        const int lane = threadIdx.x & (lanes - 1);
+        for (int i = threadIdx.x / lanes; i < INPUT_TOKENS; i += 256 / lanes)
         {
-            const bool query = unit < G;
-            f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
-            if (lane * 4 < a.dim)
-                y = delta_conv(p, r, pos0 + t, pos0, slot, unit * a.dim + lane * 4);
-            y = y * (delta_unit(y) * (query ? 1.0f / sqrtf((float)a.dim_real) : 1.0f));
-            if (lane * 4 < a.dim)
-                *reinterpret_cast<f32x4 *>((query ? p.q : p.k) + ((size_t)(query ? unit : unit - G) * p.rows + t) * a.dim + lane * 4) = y;
-        }
-        else if (unit < 2 * G + a.heads)
-        {
-            const int h = unit - 2 * G;
-            for (int d = lane * 4; d < a.vdim; d += 256)
-                *reinterpret_cast<f32x4 *>(p.v + ((size_t)h * p.rows + t) * a.vdim + d) = delta_conv(p, r, pos0 + t, pos0, slot, 2 * G * a.dim + h * a.vdim + d);
-            if (lane == 0)
-                delta_gates(a, a.d_proj + (size_t)r * a.ldp, h, p.beta[(size_t)h * p.rows + t], p.log_decay[(size_t)h * p.rows + t]);
+            const int t = blockIdx.y * INPUT_TOKENS + i, r = p.row0[e] + t;
+            if (t >= n) // (lanes of one vector leave together)
+                return;
+            if (unit < 2 * G)
+            {
+                const bool query = unit < G;
+                f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
+                if (lane * 4 < a.dim)
+                    y = delta_conv(p, r, pos0 + t, pos0, slot, unit * a.dim + lane * 4);
+                y = y * (delta_unit(y, lanes) * (query ? 1.0f / sqrtf((float)a.dim_real) : 1.0f));
+                if (lane * 4 < a.dim)
+                    *reinterpret_cast<f32x4 *>((query ? p.q : p.k) + ((size_t)(query ? unit : unit - G) * p.rows + t) * a.dim + lane * 4) = y;
+            }
+            else
+            {
+                const int h = unit - 2 * G;
+                for (int d = lane * 4; d < a.vdim; d += lanes * 4)
+                    *reinterpret_cast<f32x4 *>(p.v + ((size_t)h * p.rows + t) * a.vdim + d) = delta_conv(p, r, pos0 + t, pos0, slot, 2 * G * a.dim + h * a.vdim + d);
+                if (lane == 0)
+                    delta_gates(a, a.d_proj + (size_t)r * a.ldp, h, p.beta[(size_t)h * p.rows + t], p.log_decay[(size_t)h * p.rows + t]);
+            }
         }
     }
 
@@ -374,8 +398,12 @@ namespace llamql
         __shared__ __attribute__((aligned(16))) float s_S[16][DP + 4], s_u[16][DC + 4];
         const llam_seq_delta_args &a = p.a;
         const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
-        const int h = blockIdx.y, e = p.entry, ntok = p.ntok[e];
-        const int kv = h / (a.heads / a.kv_heads), col = blockIdx.x * 16 + c;
+        // the columns of a head read the same rows: they go to one die (blocks are dealt round robin over eight)
+        const int blocks = a.vdim / 16, h = blockIdx.x / (8 * blocks) * 8 + (blockIdx.x & 7);
+        if (h >= a.heads)
+            return;
+        const int e = p.entry, ntok = p.ntok[e];
+        const int kv = h / (a.heads / a.kv_heads), col = (blockIdx.x >> 3) % blocks * 16 + c;
         const bool fresh = p.pos[e] == 0;
         float *state = a.d_state + ((size_t)p.slot[e] * a.heads + h) * DP * a.vdim + col;
         const float *qrows = p.q + (size_t)kv * p.rows * DP;
@@ -576,7 +604,7 @@ namespace llamql
         template <int DP>
         bool walk_launch(const char *fn, const DeltaArgs &p, hipStream_t st)
         {
-            hipLaunchKernelGGL(delta_walk_kernel<DP>, dim3(p.a.vdim / 16, p.a.heads), dim3(256), 0, st, p);
+            hipLaunchKernelGGL(delta_walk_kernel<DP>, dim3(round_up(p.a.heads, 8) * (p.a.vdim / 16)), dim3(256), 0, st, p);
             return launched(fn);
         }
     } // namespace
@@ -630,7 +658,7 @@ extern "C" bool llam_seq_delta_prefill(const llam_seq_delta_args *a, const llam_
     if (!set_device(fn, device_id))
         return false;
     hipStream_t st = as_stream(stream);
-    hipLaunchKernelGGL(delta_inputs_kernel, dim3(ceil_div(2 * a->kv_heads + a->heads, 4), ntok), dim3(256), 0, st, p);
+    hipLaunchKernelGGL(delta_inputs_kernel, dim3(2 * a->kv_heads + a->heads, ceil_div(ntok, INPUT_TOKENS)), dim3(256), 0, st, p);
     if (!launched(fn))
         return false;
     if (a->taps > 1)

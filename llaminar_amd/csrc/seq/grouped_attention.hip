@@ -67,7 +67,7 @@ namespace llamql
     __device__ __forceinline__ int att_low(int i, int chunk) { return i / chunk * chunk; }
 
     template <typename T, int DK, int DV, int WR, int RG>
-    __global__ void __launch_bounds__(ATT_THREADS)
+    __global__ void __launch_bounds__(ATT_THREADS, sizeof(T) == 2 && WR == 4 && DK + DV <= 256 ? 2 : 1)
         attention_kernel(AttentionArgs p)
     {
         using O = Operand<T>;
@@ -93,7 +93,7 @@ namespace llamql
         const int e = p.first + ei, split = blockIdx.y;
         const int per = p.heads / p.groups;
         const int R = p.ntok[e] * per, pos0 = p.pos[e], row0 = p.row0[e];
-        const int rb = blockIdx.x * 16 * RG * WR;
+        const int rb = (gridDim.x - 1 - blockIdx.x) * 16 * RG * WR; // the longest walks first
         if (rb >= R)
             return;
         const int last_row = rb + 16 * RG * WR - 1 < R ? rb + 16 * RG * WR - 1 : R - 1;
@@ -420,19 +420,34 @@ namespace llamql
         int used = (pos0 + tok - low) / p.stretch + 1;
         used = used < p.nsplit ? used : p.nsplit;
         const size_t at = (size_t)blockIdx.y * p.nsplit * p.rcap + row;
-        const int team = threadIdx.x / LANES, d = threadIdx.x % LANES * 4;
-        float M = -INFINITY;
-        for (int s = 0; s < used; ++s)
-            M = fmaxf(M, p.part_ml[(at + (size_t)s * p.rcap) * 2]);
-        float L = 0.0f;
+        const int team = threadIdx.x / LANES, d = threadIdx.x % LANES * 4, lane = threadIdx.x & 63;
+        // every wavefront works out the factors, a stretch a lane
+        float M = -INFINITY, L = 0.0f;
         f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
-        for (int s = 0; s < used; ++s)
+        for (int s0 = 0; s0 < used; s0 += 64)
         {
-            const size_t k = at + (size_t)s * p.rcap;
-            const float f = expf(p.part_ml[k * 2] - M);
-            L += f * p.part_ml[k * 2 + 1];
-            if (s % TEAMS == team)
-                y = y + *reinterpret_cast<const f32x4 *>(p.part_o + k * DV + d) * f;
+            const size_t k = (at + (size_t)(s0 + lane < used ? s0 + lane : s0) * p.rcap) * 2;
+            const float m = s0 + lane < used ? p.part_ml[k] : -INFINITY, l = p.part_ml[k + 1];
+            float top = fmaxf(m, M);
+#pragma unroll
+            for (int off = 32; off > 0; off >>= 1)
+                top = fmaxf(top, __shfl_xor(top, off, 64));
+            const float base = top == -INFINITY ? 0.0f : top;
+            const float f = expf(m - base), before = expf(M - base);
+            L = L * before + wave_sum64(f * l);
+            y = y * before;
+            M = top;
+            const int n = used - s0 < 64 ? used - s0 : 64;
+            for (int s = team; s < n + team; s += 4 * TEAMS)
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                {
+                    const bool in = s + j * TEAMS < n;
+                    const int mine = in ? s + j * TEAMS : 0;
+                    const float w = __shfl(f, mine, 64);
+                    const f32x4 o = *reinterpret_cast<const f32x4 *>(p.part_o + (at + (size_t)(s0 + mine) * p.rcap) * DV + d);
+                    y = y + o * (in ? w : 0.0f);
+                }
         }
         *reinterpret_cast<f32x4 *>(&s_y[team][d]) = y;
         __syncthreads();

@@ -6,10 +6,11 @@ namespace llamql
 {
     constexpr int ROW_THREADS = 256;
 
+    constexpr int EMBED_WIDE_ROWS = 256; // rows from which a workgroup takes a whole row
     __global__ void __launch_bounds__(ROW_THREADS)
         seq_embed_kernel(llam_seq_embed_args p, const int32_t *__restrict__ ids, float *__restrict__ x, int ldx)
     {
-        const int m = blockIdx.y, id = ids[m], c = blockIdx.x * ROW_THREADS + threadIdx.x;
+        const int m = blockIdx.y, id = ids[m], last = m > 0 ? ids[m - 1] : 0;
         const bool ok = id >= 0 && id < p.vocab;
         const bf16 *table = static_cast<const bf16 *>(p.d_table), *pairs = static_cast<const bf16 *>(p.d_pairs);
         long pair = -1;
@@ -21,13 +22,31 @@ namespace llamql
                 pair = p.buckets;
             else if (pos > 0 && pos < p.cap)
             {
-                const int before = m > 0 && p.d_row_slot[m - 1] == slot ? ids[m - 1] : history[pos - 1];
-                pair = ((long)before * p.mul_prev + (long)id * p.mul_cur) % p.buckets;
+                const int before = m > 0 && p.d_row_slot[m - 1] == slot ? last : history[pos - 1];
+                const long sum = (long)before * p.mul_prev + (long)id * p.mul_cur;
+                pair = (sum >> 32) == 0 ? (long)((uint32_t)sum % (uint32_t)p.buckets) : sum % p.buckets;
             }
             if (blockIdx.x == 0 && threadIdx.x == 0 && pos >= 0 && pos < p.cap)
                 history[pos] = id;
         }
-        if (c < ldx)
+        if ((p.width & 3) == 0 && (ldx & 3) == 0)
+        {
+            // four columns at a time
+#pragma unroll 2
+            for (int c = (blockIdx.x * ROW_THREADS + threadIdx.x) * 4; c < ldx; c += gridDim.x * ROW_THREADS * 4)
+            {
+                f32x4 v = {0.0f, 0.0f, 0.0f, 0.0f};
+                if (ok && c < p.width)
+                {
+                    v = __builtin_convertvector(*reinterpret_cast<const bf16x4 *>(table + (size_t)id * p.width + c), f32x4) * p.scale;
+                    if (pair >= 0)
+                        v = v + __builtin_convertvector(*reinterpret_cast<const bf16x4 *>(pairs + (size_t)pair * p.width + c), f32x4);
+                }
+                *reinterpret_cast<f32x4 *>(x + (size_t)m * ldx + c) = v;
+            }
+            return;
+        }
+        for (int c = blockIdx.x * ROW_THREADS + threadIdx.x; c < ldx; c += gridDim.x * ROW_THREADS)
         {
             float v = 0.0f;
             if (ok && c < p.width)
@@ -448,11 +467,13 @@ extern "C" bool llam_seq_embed(const llam_seq_embed_args *a, const int32_t *d_id
         return fail(fn, "bad size (M=%d vocab=%d width=%d ldx=%d)", M, a->vocab, a->width, ldx);
     if (a->d_pairs && (!a->d_row_slot || !a->d_row_pos || !a->d_history || a->buckets < 1 || a->cap < 1))
         return fail(fn, "pairs of tokens need rows, a history and buckets=%d cap=%d of at least 1", a->buckets, a->cap);
+    if (!aligned16(a->d_table) || !aligned16(a->d_pairs) || !aligned16(d_x))
+        return fail(fn, "misaligned rows");
     if (M == 0)
         return true;
     if (!set_device(fn, device_id))
         return false;
-    hipLaunchKernelGGL(seq_embed_kernel, dim3(ceil_div(ldx, ROW_THREADS), M), dim3(ROW_THREADS), 0, as_stream(stream), *a, d_ids, d_x, ldx);
+    hipLaunchKernelGGL(seq_embed_kernel, dim3(M >= EMBED_WIDE_ROWS ? 1 : ceil_div(ldx, 4 * ROW_THREADS), M), dim3(ROW_THREADS), 0, as_stream(stream), *a, d_ids, d_x, ldx);
     return launched(fn);
 }
 

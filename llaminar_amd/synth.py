@@ -57,10 +57,11 @@ def gemv_bytes(fmt: int, N: int, K: int, M: int = 1) -> int:
 
 
 def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap: int, max_rows: int = 2048,
-                         dtype: str = "bfloat16", eps: float = 1e-5, seed: int = 0):
+                         dtype: str = "bfloat16", eps: float = 1e-5, seed: int = 0, pairs: int = 0):
     """A sequence.SequenceModel of random bf16 weights made on the device (matrices too big to build on the host
     every run).  ``layers``: sequence.Layer descriptions with sizes only; every tensor is filled in here, N(0, 1/in)
-    (random weights need no particular order of tiles).  The tensors live as long as the model."""
+    (random weights need no particular order of tiles).  ``pairs``: buckets of an embedding of token pairs.  The tensors
+    live as long as the model."""
     import ctypes
 
     import torch
@@ -86,14 +87,16 @@ def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap
         return t.data_ptr(), t.numel() * 2
 
     def vector(n, value=1.0):
-        t = torch.full((n,), value, device=device)
+        t = torch.full((n,), value, device=device) if isinstance(value, float) else value.to(device)
         model.keep.append(t)
         return t.data_ptr()
 
     for n, w in enumerate(layers):
         H, d, v, wp, read = w.heads, P(w.dim), P(w.vdim), P(width), 0
+        if w.mixer == sq.MIXER_ATTENTION:
+            d, v = sq.A(w.dim), sq.A(w.vdim)
         w.norm1 = vector(wp)
-        w.w_out, b = matrix(wp, H * v)
+        w.w_out, b = matrix(wp, H * v + (P(w.ff) if w.parallel and w.ffn else 0))
         read += b
         if w.mixer == sq.MIXER_LATENT_ATTENTION:
             own = w.kv_from < 0
@@ -104,6 +107,16 @@ def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap
             read += b1 + b2 + b3 + b4
             w.q_norm, w.kv_norm = vector(P(w.q_rank)), vector(P(w.kv_rank))
             w.scale = w.scale or w.dim ** -0.5
+        elif w.mixer == sq.MIXER_ATTENTION:
+            w.w_in, b = matrix(H * d + (w.kv_heads * (d + v) if w.kv_from < 0 else 0), wp)
+            read += b
+            w.scale, w.rot_dims = w.scale or w.dim ** -0.5, w.rot_dims or w.dim
+            w.turns = vector(w.rot_dims // 2, 10000.0 ** (-torch.arange(0, w.rot_dims, 2, dtype=torch.float64) / w.rot_dims) / 6.283185307179586)
+        elif w.mixer == sq.MIXER_DELTA:
+            w.w_in, b = matrix(2 * w.kv_heads * d + 2 * H * v + 2 * H, wp)
+            read += b
+            w.conv = vector(w.taps * (2 * w.kv_heads * d + H * v), 0.5)
+            w.a_log, w.dt_bias, w.head_norm = vector(H, -2.0), vector(H, -1.0), vector(v)
         else:
             w.w_in, b = matrix(2 * H * (d + v) + 2 * H, wp)
             read += b
@@ -111,10 +124,12 @@ def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap
             w.gate_cap, w.scale = w.gate_cap or 15.0, w.dim ** -0.5
         if w.ffn:
             w.norm2 = vector(wp)
-        if w.ffn == sq.FFN_GATED:
+        if w.ffn in (sq.FFN_GATED, sq.FFN_GATED_CLAMP):
             w.w_up, b1 = matrix(2 * P(w.ff), wp)
-            w.w_down, b2 = matrix(wp, P(w.ff))
-            read += b1 + b2
+            read += b1
+            if not w.parallel:
+                w.w_down, b2 = matrix(wp, P(w.ff))
+                read += b2
         elif w.ffn == sq.FFN_EXPERTS:
             w.w_up, b1 = matrix(P(w.ff), wp, w.experts)
             w.w_down, b2 = matrix(wp, P(w.ff), w.experts)
@@ -133,5 +148,11 @@ def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap
     head, b = matrix(vocab, P(width))
     model.weight_bytes.append(b)
     torch.cuda.synchronize()
-    model._check(model.L.llam_seqm_set_globals(model.h, ctypes.byref(sq.Globals(embed.data_ptr(), vector(P(width)), head, 1.0))))
+    g_ = sq.Globals(embed.data_ptr(), vector(P(width)), head, 1.0)
+    if pairs:
+        table = torch.randn(pairs + 1, width, device=device, generator=g).to(torch.bfloat16)
+        model.keep.append(table)
+        g_.pairs, g_.buckets, g_.mul_prev, g_.mul_cur = table.data_ptr(), pairs, 31, 7
+    torch.cuda.synchronize()
+    model._check(model.L.llam_seqm_set_globals(model.h, ctypes.byref(g_)))
     return model

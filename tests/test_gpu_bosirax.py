@@ -80,6 +80,16 @@ def test_attention_over_a_cache(dev, case, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("vdim", [64, 128, 256])
+@pytest.mark.parametrize("dim", [64, 128, 256])
+def test_attention_at_every_padded_size(dev, dim, vdim, dtype):
+    """Rows that the wavefronts share (decoding) and rows of their own (prompts), across a chunk's edge."""
+    attend(dev, dtype, 4, 2, dim, vdim, 1, 0, 333)
+    attend(dev, dtype, 6, 2, dim, vdim, 5, 90, 177)
+    attend(dev, dtype, 6, 2, dim, vdim, 150, 90, 40)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("case", [(8, 2, 64, 64, 1, 100, 1000, 128), (4, 2, 128, 64, 60, 69, 1003, 128), (4, 4, 64, 128, 100, 150, 2040, 256)], ids=str)
 def test_attention_over_a_ring_that_has_gone_round(dev, case, dtype):
     attend(dev, dtype, *case)
