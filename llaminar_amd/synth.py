@@ -152,7 +152,7 @@ def sequence_model_torch(layers, width: int, vocab: int, device, slots: int, cap
     if pairs:
         table = torch.randn(pairs + 1, width, device=device, generator=g).to(torch.bfloat16)
         model.keep.append(table)
-        g_.pairs, g_.buckets, g_.mul_prev, g_.mul_cur = table.data_ptr(), pairs, 31, 7
+        g_.pairs, g_.buckets, g_.mul_prev, g_.mul_cur = table.data_ptr(), pairs, 40503, 19
     torch.cuda.synchronize()
     model._check(model.L.llam_seqm_set_globals(model.h, ctypes.byref(g_)))
     return model
